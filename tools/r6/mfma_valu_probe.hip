@@ -52,7 +52,6 @@ __global__ __launch_bounds__(512) void probe(float * out, unsigned long long * c
                 if (KIND == 9) asm volatile("v_pk_mul_f16 %0, %0, %1" : "+v"(v0) : "v"(v2));
                 if (KIND == 10) asm volatile("v_lshrrev_b32 %0, 4, %0" : "+v"(v0));
                 if (KIND == 11) asm volatile("v_fma_f16 %0, %0, %1, %2" : "+v"(v0) : "v"(v2), "v"(v3));
-                if (KIND == 12) asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(*(unsigned long long *) &cyc[0]) : "v"(0ull), "v"(0ull));
             }
         }
     }
