@@ -30,7 +30,9 @@ EXTRA = os.environ.get("PM355_EXTRA_FLAGS", "").split()
 # (mmvq.hip hands the six values its prologue starts with that way: +0.4 % on the 70B decode step, +0.9 % on the 8B one, interleaved A/B on one box).
 # The option is an internal LLVM one: it goes to mmvq.hip only, and only when this compiler accepts it (probed once; a ROCm / LLVM upgrade that renames it
 # builds without it instead of failing everything).
-FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fvisibility=hidden",
+# -packed-fp32-ops: some v_pk_*_f32 forms the backend makes from ordinary float code have given wrong results on these GPUs (hipcc's host pass warns that it
+# does not know the feature: harmless).
+FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fvisibility=hidden", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
          "-Wall", "-Wno-unused-const-variable", "-Wno-unused-value", "-Wno-unused-function", "-Wno-unused-result"]
 KERNARG_PRELOAD = ["-mllvm", "-amdgpu-kernarg-preload-count=16"]
 # (round 5: first restricted to mmvq.hip - the 2..64-token steps, ten small launches per layer, then ran 1.3-2.4 % slower than round 4's: every kernel of the
