@@ -32,7 +32,7 @@ extern "C" {
 
 /* ggml type ids, identical to enum ggml_type (ggml/include/ggml.h:356-372) */
 enum { PM355_TYPE_F32 = 0, PM355_TYPE_F16 = 1, PM355_TYPE_Q8_0 = 8, PM355_TYPE_Q4_K = 12,
-       PM355_TYPE_Q5_K = 13, PM355_TYPE_Q6_K = 14 };
+       PM355_TYPE_Q5_K = 13, PM355_TYPE_Q6_K = 14, PM355_TYPE_BF16 = 30 };
 
 enum { PM355_OK = 0, PM355_E_UNSUPPORTED = -1, PM355_E_SHAPE = -2, PM355_E_ALIGN = -3, PM355_E_RANGE = -4,
        PM355_E_HIP = -10, PM355_E_NOMEM = -11 };
@@ -416,7 +416,7 @@ PM355_API int pm355_op_get_rows_f32(const pm355_tensor * a, const int32_t * d_id
 typedef struct pm355_model pm355_model;
 
 typedef struct {                          /* llm_load_hparams (src/llama.cpp:5823) subset */
-    int32_t arch;                         /* 0 = llama (rope NORM, optional rope_freqs), 1 = qwen2 (rope NEOX, qkv bias) */
+    int32_t arch;                         /* pm355_arch_id(): 0 = llama (rope NORM, optional rope_freqs), 1 = qwen2 (rope NEOX, qkv bias) */
     int32_t n_layer, n_embd, n_head, n_head_kv, head_dim, n_ff, n_vocab, n_ctx, n_ctx_orig;
     float   rms_eps, rope_freq_base, rope_freq_scale;
     int32_t pad_;
@@ -424,8 +424,68 @@ typedef struct {                          /* llm_load_hparams (src/llama.cpp:582
 
 enum pm355_tensor_kind { PM355_T_ATTN_NORM = 0, PM355_T_WQ, PM355_T_WK, PM355_T_WV, PM355_T_WO, PM355_T_FFN_NORM,
                          PM355_T_FFN_GATE, PM355_T_FFN_UP, PM355_T_FFN_DOWN, PM355_T_BQ, PM355_T_BK, PM355_T_BV,
-                         PM355_T_TOK_EMBD, PM355_T_OUT_NORM, PM355_T_OUTPUT, PM355_T_ROPE_FREQS, PM355_T_COUNT };
+                         PM355_T_TOK_EMBD, PM355_T_OUT_NORM, PM355_T_OUTPUT, PM355_T_ROPE_FREQS,
+                         /* layer-described models; ATTN_NORM / FFN_NORM / OUT_NORM are the weights of the norms whose biases these are */
+                         PM355_T_ATTN_NORM_B, PM355_T_FFN_NORM_B, PM355_T_OUT_NORM_B, PM355_T_W_OUT_GATE, PM355_T_SINK, PM355_T_VALUE_MIX, PM355_T_FFN_UP_B,
+                         PM355_T_FFN_DOWN_B, PM355_T_COUNT };
 enum { PM355_HAS_EMBD = 1, PM355_HAS_HEAD = 2 };
+
+/* Architectures are looked up by name ("llama", "qwen2", "kudirax"): the id for pm355_hparams.arch / pm355_stack_desc.arch, or PM355_E_UNSUPPORTED where this build
+ * does not carry the implementation. */
+PM355_API int pm355_arch_id(const char * name);
+
+/* ---- (B') layer-described models ------------------------------------------------------------------------------------------------
+ * A model given layer by layer (csrc/stack.hip): sizes and constants may differ between layers, weights are dense (bf16, or f32 for a model that computes in 32-bit
+ * throughout), and the KV cache is a pool of 64-token pages shared by the open sequences. Tensors are set through pm355_model_set_tensor like any other model's
+ * (BF16 or F32 host data, row-major [out][in]); the head, residual stream, attention weights and norms are f32. The mechanisms of a layer are flags and constants: */
+enum { PM355_MIX_QK_NORM    = 1,        /* q and k divided by their root mean square over the head, per head, no weight */
+       PM355_MIX_SINK       = 2,        /* exp(sink[head]) joins the softmax denominator: no key, no value, neither scaled nor capped */
+       PM355_MIX_VALUE_MIX  = 4,        /* v <- (1 - lambda) v + lambda v_first; v_first = v of the first layer with this flag, same token; the mix is what is cached */
+       PM355_MIX_OUT_GATE   = 8 };      /* heads multiplied by sigmoid(W_g h) before the output projection */
+enum { PM355_MASK_CAUSAL = 0, PM355_MASK_CHUNK = 1 };      /* CHUNK: i sees j <= i with floor(i / size) == floor(j / size), counted from position 0 of the sequence */
+enum { PM355_FF_NONE = 0, PM355_FF_DENSE = 1 };            /* W_down act(W_up h + b_up) + b_down */
+enum { PM355_ACT_NONE = 0, PM355_ACT_RELU2 = 1 };          /* square of relu */
+typedef struct {
+    int32_t n_head, n_head_kv, k_dim, v_dim;   /* query head h reads KV head h / (n_head / n_head_kv) */
+    int32_t mix_flags, mask, mask_size;
+    float   scale, softcap;                    /* score = (q . k) * scale, then softcap * tanh(score / softcap) when softcap > 0 */
+    int32_t ff, n_ff, act;
+} pm355_layer_spec;
+typedef struct {
+    int32_t arch, n_layer, n_embd, n_vocab;
+    int32_t type;                              /* PM355_TYPE_BF16: bf16 products with f32 accumulation; PM355_TYPE_F32: everything in 32-bit */
+    float   norm_eps;
+    const pm355_layer_spec * layers;           /* n_layer of them; norms are layer norms with weight and bias on each sublayer's OUTPUT: x + norm(sublayer(x)) */
+} pm355_stack_desc;
+PM355_API pm355_model * pm355_model_new_stack(const pm355_stack_desc * d);
+
+/* ---- (B") sequences and batches: every architecture --------------------------------------------------------------------------------
+ * pm355_model_finalize_pool: cache for n_seq open sequences that hold at most pool_tokens tokens together (each rounded up to whole pages; layer windows: one slab of
+ * n_ctx cells per sequence instead) and scratch for max_tokens tokens at once (longer batches run in pieces).
+ * pm355_model_batch: one step over the entries - prompt portions of any length next to single decoded tokens - all of them in one pass where the architecture has a
+ * batched step (layer-described models). d_logits: f32 [wanted rows][n_vocab] in the order of entries and of `want`; d_argmax: int32 per wanted row (greedy token,
+ * first maximum); either may be NULL. tokens: host pointer; NULL = one token, the sequence's last greedy token, taken on the device. Asynchronous; the host arrays may
+ * be reused on return. Errors are detected before anything is changed: PM355_E_NOMEM when the pages do not suffice. */
+typedef struct { int32_t seq, n_tokens; const int32_t * tokens; int32_t n_want; const int32_t * want; } pm355_batch_entry;
+typedef struct { int32_t page_tokens, n_pages, free_pages, n_seqs, free_seqs, max_seq_tokens; } pm355_pool_info;
+PM355_API int pm355_model_finalize_pool(pm355_model * m, int max_tokens, int n_seq, int64_t pool_tokens);
+PM355_API int pm355_model_seq_new(pm355_model * m);                 /* sequence id >= 0, or PM355_E_NOMEM */
+PM355_API int pm355_model_seq_free(pm355_model * m, int seq);       /* its pages / slab go back to the pool */
+PM355_API int pm355_model_seq_len(pm355_model * m, int seq);        /* tokens processed so far */
+PM355_API int pm355_model_pool_info(pm355_model * m, pm355_pool_info * out);
+PM355_API int pm355_model_batch(pm355_model * m, const pm355_batch_entry * entries, int n_entries, float * d_logits, int32_t * d_argmax, pm355_stream_t stream);
+PM355_API int pm355_model_n_vocab(const pm355_model * m);
+
+/* The page pool by itself (host only, no device): what pm355_model_batch allocates from. pages of 64 tokens; a sequence's table maps page index -> pool page or -1. */
+typedef struct pm355_page_pool pm355_page_pool;
+PM355_API pm355_page_pool * pm355_page_pool_new(int n_pages, int n_seqs, int max_seq_pages);
+PM355_API void pm355_page_pool_free(pm355_page_pool * p);
+PM355_API int pm355_page_pool_open(pm355_page_pool * p);                                  /* sequence id or PM355_E_NOMEM */
+PM355_API int pm355_page_pool_close(pm355_page_pool * p, int seq);
+PM355_API int pm355_page_pool_grow(pm355_page_pool * p, int seq, int n_tokens);           /* pages for positions [0, n_tokens) that are not there yet; all or nothing */
+PM355_API int pm355_page_pool_drop_before(pm355_page_pool * p, int seq, int position);    /* releases the pages that lie wholly in front of `position` */
+PM355_API int pm355_page_pool_page(const pm355_page_pool * p, int seq, int index);
+PM355_API int pm355_page_pool_free_pages(const pm355_page_pool * p);
 
 /* A model holds the tensors of layers [layer_lo, layer_hi) — the window prima.cpp's piped-ring assigns to this
  * rank (this_layer_is_mine, src/llama.cpp:3838-3852) — plus tok_embd (HAS_EMBD) and output_norm/output (HAS_HEAD). */

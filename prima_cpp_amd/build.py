@@ -4,6 +4,7 @@ machinery: the .so travels with the repo snapshot to the GPU box.
 build()            the product library prima_cpp_amd/libprima_mi355.so
 build_experiments()  libprima_mi355_exp.so = the product sources + decode_engine.hip with -DPM_EXPERIMENTS=1: round 5's three measured-slower forms of the decode
                    layer live only there (tests/test_gpu_experiments.py runs their tests against it)
+build_dense()      libprima_mi355_dense.so = the sources a layer-described model needs (seconds instead of minutes); same C ABI, the other architectures are not registered
 build_probe()      tools/csrc -> prima_cpp_amd/libprima_mi355_probe.so: measurement helpers (HBM streaming-read ceiling, persistent-layer
                    skeleton) that bench.py / tools/ load separately - nothing of them is inside the product library
 build(tag=, extra=)  an A/B or measurement variant of the product library with extra compiler flags -> ab/<tag>.so, objects under
@@ -16,9 +17,12 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 ROOT = os.path.dirname(HERE)
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libprima_mi355.so")
+DENSE_LIB = os.path.join(HERE, "libprima_mi355_dense.so")
 PROBE_LIB = os.path.join(HERE, "libprima_mi355_probe.so")
-SOURCES = ["c_api.hip", "quantize.hip", "mmvq.hip", "mmvq_cols.hip", "repack.hip", "layer_ops.hip", "ggml_ops.hip", "engine.hip", "mmq.hip", "mmq_pf.hip", "mmq_i8.hip", "mmq_big.hip",
-           "attn_prefill.hip", "attn_cached.hip", "attn_flash_mfma.hip", "attn_split.hip", "attn_flash.hip", "attn_q8.hip", "ring.hip", "upload.hip", "ts.hip"]
+# what a layer-described (dense-weight) model needs: also a library of its own, so that such a model can be served without compiling the quantized kernels
+DENSE_SOURCES = ["c_api_base.hip", "model.hip", "kv_pool.hip", "stack.hip", "dense_small.hip", "dense_gemm.hip", "dense_ops.hip", "attn_paged.hip", "repack.hip", "upload.hip"]
+SOURCES = DENSE_SOURCES + ["c_api.hip", "quantize.hip", "mmvq.hip", "mmvq_cols.hip", "layer_ops.hip", "ggml_ops.hip", "engine.hip", "mmq.hip", "mmq_pf.hip", "mmq_i8.hip", "mmq_big.hip",
+           "attn_prefill.hip", "attn_cached.hip", "attn_flash_mfma.hip", "attn_split.hip", "attn_flash.hip", "attn_q8.hip", "ring.hip", "ts.hip"]
 # round 5's measured-slower forms of the decode layer (sum-of-squares partials, attention tail, persistent engine): a library of their own, loaded by their tests
 EXP_LIB = os.path.join(HERE, "libprima_mi355_exp.so")
 EXP_SOURCES = SOURCES + ["decode_engine.hip"]
@@ -77,7 +81,7 @@ def _compile(srcs, hdrs, objdir, lib, flags, force, verbose):
             if verbose:
                 print(" ".join(cmd), flush=True)
             procs.append((cmd, subprocess.Popen(cmd)))
-            if len(procs) >= (os.cpu_count() or 4):
+            if len(procs) >= min(os.cpu_count() or 4, int(os.environ.get("MAX_JOBS") or 16)):
                 c, pr = procs.pop(0)
                 if pr.wait():
                     raise subprocess.CalledProcessError(pr.returncode, c)
@@ -102,6 +106,11 @@ def build(force=False, verbose=False, tag=None, extra=()):
         ab = os.path.join(ROOT, "ab")
         return _compile(srcs, _headers(), os.path.join(ab, "obj_" + tag), os.path.join(ab, tag + ".so"), EXTRA + list(extra) + FLAGS, force, verbose)
     return _compile(srcs, _headers(), CSRC, LIB, EXTRA + FLAGS, force, verbose)
+
+
+def build_dense(force=False, verbose=False):
+    srcs = [os.path.join(CSRC, s) for s in DENSE_SOURCES]
+    return _compile(srcs, _headers(), CSRC, DENSE_LIB, EXTRA + FLAGS, force, verbose)
 
 
 def build_experiments(force=False, verbose=False):

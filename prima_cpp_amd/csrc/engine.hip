@@ -13,6 +13,7 @@
 #include "pm355_kernels.h"
 #include "pm355_layer_ops.h"
 #include "pm355_engine.h"
+#include "pm355_model.h"
 #include <math.h>
 #include <stdio.h>
 #include <string.h>
@@ -31,7 +32,7 @@ struct Slot { void * d[12] = {}; hipEvent_t ready = nullptr, free_ = nullptr; in
 
 } // namespace
 
-struct pm355_model {
+struct pm_window : pm355_model {
     pm355_hparams hp;
     int lo, hi, flags;
     std::vector<Layer> layers;            // hi - lo
@@ -103,12 +104,42 @@ struct pm355_model {
     // captured single-token step graphs, keyed on everything that is baked into the kernel arguments
     struct StepGraph { const void * in, * tok; void * out, * logits, * argmax; int adv, rot, head, regime; hipGraphExec_t exec; };
     std::vector<StepGraph> graphs;
-    char err[256];
+    // batches: open sequences (a sequence holds one KV slab), their last greedy token on the device, and the hidden rows of a portion whose logits are asked for
+    std::vector<char> seq_open; int32_t * d_last = nullptr; float * rows = nullptr;
+
+    ~pm_window() override;
+    int set_tensor(int kind, int layer, int type, const void * host, size_t nbytes) override;
+    int fill_tensor(int kind, int layer, int type, uint64_t seed, float scale) override;
+    void * tensor_ptr(int kind, int layer, int * type_out) override;
+    int set_streaming(int n) override;
+    uint64_t streamed() const override { return streamed_bytes; }
+    int finalize(int max_tokens_, int n_seq_) override;
+    int finalize_pool(int max_tokens_, int n_seq_, int64_t pool_tokens) override;
+    size_t weight_bytes() const override;
+    size_t kv_bytes_per_pos() const override;
+    int kv_clear(hipStream_t st) override;
+    void * kv_ptr(int layer, int which) override;
+    int n_embd() const override { return hp.n_embd; }
+    int n_vocab() const override { return hp.n_vocab; }
+    int n_seqs() const override { return n_seq; }
+    int check() override;
+    int seq_new() override;
+    int seq_free(int seq) override;
+    int seq_len(int seq) override;
+    int pool_info(pm355_pool_info * out) override;
+    int batch(const pm355_batch_entry * e, int n, float * d_logits, int32_t * d_argmax, hipStream_t st) override;
+    int decode(int seq, const int32_t * d_tokens, const float * d_x_in, int T, int pos0, float * d_x_out, float * d_logits, int32_t * d_argmax, hipStream_t st) override;
+    int set_seq_pos(int seq, int pos, hipStream_t st) override;
+    int set_seq(int seq, hipStream_t st) override;
+    int head(const float * d_x_row, float * d_logits, int32_t * d_argmax, hipStream_t st) override;
+    int step_ex(const int32_t * d_token, const float * d_x_in, float * d_x_out, float * d_logits, int32_t * d_argmax, int advance, int rotate, int head_first, int use_graph,
+                hipStream_t st) override;
+    int generate(int32_t * d_io, int pos0, int n_steps, int use_graph, hipStream_t st) override;
 };
 
 namespace {
 
-int tensor_shape(const pm355_model * m, int kind, int64_t & K, int64_t & N) {
+int tensor_shape(const pm_window * m, int kind, int64_t & K, int64_t & N) {
     const pm355_hparams & h = m->hp;
     const int64_t E = h.n_embd, Eq = (int64_t) h.head_dim * h.n_head, Ekv = (int64_t) h.head_dim * h.n_head_kv, F = h.n_ff;
     switch (kind) {
@@ -126,7 +157,7 @@ int tensor_shape(const pm355_model * m, int kind, int64_t & K, int64_t & N) {
     return -1;
 }
 
-Tensor * tensor_slot(pm355_model * m, int kind, int layer) {
+Tensor * tensor_slot(pm_window * m, int kind, int layer) {
     if (kind < 12) {
         if (layer < m->lo || layer >= m->hi) return nullptr;
         return &m->layers[layer - m->lo].t[kind];
@@ -140,17 +171,12 @@ Tensor * tensor_slot(pm355_model * m, int kind, int layer) {
     return nullptr;
 }
 
-int seterr(pm355_model * m, int code, const char * msg) {
-    const hipError_t e = hipGetLastError();        // also clears the sticky error
-    if (code == PM355_E_HIP) snprintf(m->err, sizeof(m->err), "%s: %s", msg, hipGetErrorString(e));
-    else snprintf(m->err, sizeof(m->err), "%s", msg);
-    return code;
-}
+int seterr(pm_window * m, int code, const char * msg) { return m->fail(code, msg); }
 // hipGetLastError() is sticky across unrelated earlier calls: test-and-clear around OUR launches only
 bool hip_ok() { return hipGetLastError() == hipSuccess; }
 
 size_t g_last_hbm = 0;        // HBM bytes of the tensor alloc_tensor allocated last (single-threaded loader)
-int alloc_tensor(pm355_model * m, Tensor * t, int kind, int type) {
+int alloc_tensor(pm_window * m, Tensor * t, int kind, int type) {
     int64_t K, N;
     if (tensor_shape(m, kind, K, N)) return PM355_E_UNSUPPORTED;
     const size_t rb = pm_weight_row_bytes(type, K);
@@ -234,7 +260,7 @@ namespace {
 
 // ---- window streaming ------------------------------------------------------------------------------------------------------------
 // enqueue the H2D copies of layer `il` into its slot on the copy stream (after the slot was released by its previous user)
-void stream_prefetch(pm355_model * m, int il, int slot) {
+void stream_prefetch(pm_window * m, int il, int slot) {
     const int n = m->hi - m->lo;
     Slot & S = m->slots[slot];
     Layer & L = m->layers[il - m->lo];
@@ -248,7 +274,7 @@ void stream_prefetch(pm355_model * m, int il, int slot) {
     (void) n;
 }
 // the layer as the kernels see it: resident tensors, or (streaming) the slot's copies once the copy stream has delivered them
-Layer layer_acquire(pm355_model * m, int il, hipStream_t st) {
+Layer layer_acquire(pm_window * m, int il, hipStream_t st) {
     Layer L = m->layers[il - m->lo];
     if (!m->n_slots) return L;
     // slots are dealt out by a running step counter, not by layer index: with n % n_slots != 0 a layer-indexed slot made the layer
@@ -262,7 +288,7 @@ Layer layer_acquire(pm355_model * m, int il, hipStream_t st) {
 }
 // the layer's last kernel has been enqueued: release its slot and start fetching the layer that uses the slot next (wrapping around
 // to the first layers of the next token)
-void layer_release(pm355_model * m, int il, hipStream_t st) {
+void layer_release(pm_window * m, int il, hipStream_t st) {
     if (!m->n_slots) return;
     const int n = m->hi - m->lo;
     const int slot = (int) (m->stream_step % (uint64_t) m->n_slots);
@@ -286,13 +312,13 @@ const int MMQ_MAX_TOKENS = [] { const char * e = getenv("PM355_MMQ_MAX_TOKENS");
 const int SMALL_ATTN_MFMA_MIN = [] { const char * e = getenv("PM355_SMALL_ATTN_MFMA_MIN"); return e ? atoi(e) : 16; }();
 const int MMQ_MULTI_MIN_TOKENS = 2;       // the fused wq | wk | wv and ffn_gate | ffn_up launches already win at 2 tokens (3 / 4 mat-vec launches otherwise)
 // the table output of the Q8_K quantizers, when this batch size takes the small-batch mat-mul (mmq_i8.hip)
-pm_q8k_tables mmq_tables(const pm355_model * m, int K, int T, hipStream_t st) {
+pm_q8k_tables mmq_tables(const pm_window * m, int K, int T, hipStream_t st) {
     pm_q8k_tables tb;
     const bool on = T >= (m->no_multi ? MMQ_MIN_TOKENS : MMQ_MULTI_MIN_TOKENS) && T <= MMQ_MAX_TOKENS && !m->no_mmq;
     if (on && pm_mmq_i8_tables(K, st, &tb) != 0) tb = pm_q8k_tables();
     return on ? tb : pm_q8k_tables();
 }
-ActQ quantize_for(pm355_model * m, const float * src, int K, int T, const Tensor * const * ws, int nw, hipStream_t st) {
+ActQ quantize_for(pm_window * m, const float * src, int K, int T, const Tensor * const * ws, int nw, hipStream_t st) {
     ActQ a; bool need_k = false, need_0 = false;
     for (int i = 0; i < nw; ++i) if (ws[i] && ws[i]->d) { if (ws[i]->type == PM_Q8_0) need_0 = true; else need_k = true; }
     if (need_k) { const pm_q8k_tables tb = mmq_tables(m, K, T, st); pm_launch_quantize_q8k(src, m->aq_k, K, T, st, tb); a.k = m->aq_k; a.tab = tb.base != nullptr; }
@@ -300,7 +326,7 @@ ActQ quantize_for(pm355_model * m, const float * src, int K, int T, const Tensor
     return a;
 }
 
-ActQ norm_quantize_for(pm355_model * m, const float * src, const float * w, int K, int T, const Tensor * const * ws, int nw, hipStream_t st) {
+ActQ norm_quantize_for(pm_window * m, const float * src, const float * w, int K, int T, const Tensor * const * ws, int nw, hipStream_t st) {
     bool need_0 = false;
     for (int i = 0; i < nw; ++i) if (ws[i] && ws[i]->d && ws[i]->type == PM_Q8_0) need_0 = true;
     if (!need_0) {
@@ -322,7 +348,7 @@ int gemv(const Tensor & w, const Tensor * w2, const ActQ & a, int T, float * y, 
 // 3..MMQ_MAX_TOKENS (32; on request 64) tokens: one pass over the weights per 32 tokens on the integer matrix cores (mmq_i8.hip) where the type / shape is served, else the mat-vec
 // (one to three passes per 8 columns). `prepped`: the kernel's activation tables already describe THIS activation set (set by the first
 // served call, cleared by the caller whenever the activations change)
-int matmul_small(pm355_model * m, const Tensor & w, const ActQ & a, int T, float * y, const float * bias, const float * resid, bool & prepped, hipStream_t st) {
+int matmul_small(pm_window * m, const Tensor & w, const ActQ & a, int T, float * y, const float * bias, const float * resid, bool & prepped, hipStream_t st) {
     // (3 / 4 tokens on the 4-slot multi-column mat-vec - two rows per activation fetch: ffn_down Q6_K 46 us - measured against this kernel once it had
     //  its operand-ordered activation table (54 us without the prologue launch): 177 vs 172 us per layer, so the matrix-core kernel keeps them)
     const bool q80 = w.type == PM_Q8_0;                  // Q8_0 weights take Q8_0 activations; the kernel builds their tables per call
@@ -337,7 +363,7 @@ int matmul_small(pm355_model * m, const Tensor & w, const ActQ & a, int T, float
 // single-token fused GEMV launch helper: jobs share the f32 activation `xf` (rms_norm'ed with norm_w when given)
 // ss_out: this launch leaves its per-workgroup sum-of-squares partials there and *n_ss_out receives their number (0: not served - the consumer
 // then reduces the row itself); ss_in / n_ss_in: partials of xf's sum of squares left by the producing launch
-int gemv_f32(pm355_model * m, const Tensor * const * ws, const Tensor * const * w2s, float * const * ys,
+int gemv_f32(pm_window * m, const Tensor * const * ws, const Tensor * const * w2s, float * const * ys,
              const float * const * biases, const float * const * resids, int nj,
              const float * xf, const float * norm_w, hipStream_t st, const pm_qkv_epi * epi = nullptr,
              double * ss_out = nullptr, int * n_ss_out = nullptr, const double * ss_in = nullptr, int n_ss_in = 0) {
@@ -357,7 +383,7 @@ int gemv_f32(pm355_model * m, const Tensor * const * ws, const Tensor * const * 
 }
 
 // result_norm + lm_head (+ greedy argmax) on ONE hidden row (build_llama's last sub-graph, src/llama.cpp:11191-11215)
-int run_head(pm355_model * m, const float * x_row, float * d_logits, int32_t * d_argmax, hipStream_t st, const double * ss_in = nullptr, int n_ss_in = 0) {
+int run_head(pm_window * m, const float * x_row, float * d_logits, int32_t * d_argmax, hipStream_t st, const double * ss_in = nullptr, int n_ss_in = 0) {
     if (!m->output.d || !m->out_norm.d) return seterr(m, PM355_E_UNSUPPORTED, "head: output / output_norm missing");
     const Tensor * ow[1] = {&m->output};
     float * lg = d_logits ? d_logits : m->logits;
@@ -377,7 +403,7 @@ int run_head(pm355_model * m, const float * x_row, float * d_logits, int32_t * d
 // nullptr: this window is not served (types, shapes, streaming, long-context regime) - the caller takes the five-launch path.
 // may_build = false (the stream is being captured: no allocation, no synchronous copy): only a plan that exists already is returned.
 #if PM_EXPERIMENTS
-pm355_model::EnginePlan * engine_plan_for(pm355_model * m, const float * cur, float * d_x_out, bool may_build = true) {
+pm_window::EnginePlan * engine_plan_for(pm_window * m, const float * cur, float * d_x_out, bool may_build = true) {
     for (auto & e : m->eng_plans) if (e.in == cur && e.out == d_x_out) return &e;
     if (m->eng_refused || !may_build) return nullptr;
     const float * in0 = cur;
@@ -392,7 +418,7 @@ pm355_model::EnginePlan * engine_plan_for(pm355_model * m, const float * cur, fl
     float * act = nullptr;
     if (hipMalloc((void **) &act, per_bytes * (size_t) nl + 256 * sizeof(double) + 256) != hipSuccess) { (void) hipGetLastError(); m->eng_refused = true; return nullptr; }
     pm_eng_plan * pl = pm_eng_plan_new();
-    auto refuse = [&](const char * why, int rc) -> pm355_model::EnginePlan * {
+    auto refuse = [&](const char * why, int rc) -> pm_window::EnginePlan * {
         if (getenv("PM355_ENGINE_VERBOSE")) fprintf(stderr, "prima_mi355 engine: not served (%s, rc %d) - five launches per layer\n", why, rc);
         (void) hipGetLastError();
         pm_eng_plan_free(pl); (void) hipFree(act); m->eng_refused = true; return nullptr;
@@ -457,15 +483,15 @@ pm355_model::EnginePlan * engine_plan_for(pm355_model * m, const float * cur, fl
 }
 
 #else
-pm355_model::EnginePlan * engine_plan_for(pm355_model *, const float *, float *, bool = true) { return nullptr; }      // (experiments library only)
+pm_window::EnginePlan * engine_plan_for(pm_window *, const float *, float *, bool = true) { return nullptr; }      // (experiments library only)
 #endif
-bool engine_eligible(const pm355_model * m) {
+bool engine_eligible(const pm_window * m) {
     return m->use_engine && !m->no_fuse && !m->long_ctx && !m->n_slots && m->ss && m->qkv_epi && m->rope_tab && (m->rope.mode == 0 || m->rope.mode == 2) && m->hi > m->lo;
 }
 
 // which single-token attention path the current sequence takes: 0 = one workgroup per head; else the cells the long-context grid is
 // sized for (power-of-two bucket >= position + 1, capped at n_ctx) - also the key of the captured step graph
-int attn_regime(const pm355_model * m) {
+int attn_regime(const pm_window * m) {
     const int pos = m->h_pos[m->h_seq];
     if (!m->split_scratch || pos < m->split_min) return 0;
     long b = 1024;
@@ -475,7 +501,7 @@ int attn_regime(const pm355_model * m) {
 
 // the single-token layer sequence (5 launches per layer)
 // *n_ss_end: number of partials the LAST layer's ffn_down left in m->ss + 256 for the sum of squares of the window's output row (0: none)
-int run_layers_fused(pm355_model * m, const float * cur, float * d_x_out, const float ** cur_out, hipStream_t st, int * n_ss_end = nullptr) {
+int run_layers_fused(pm_window * m, const float * cur, float * d_x_out, const float ** cur_out, hipStream_t st, int * n_ss_end = nullptr) {
     const pm355_hparams & hp = m->hp;
     const int H = hp.n_head, Hkv = hp.n_head_kv, dh = hp.head_dim;
     const float kq_scale = 1.0f / sqrtf((float) dh);
@@ -576,7 +602,7 @@ int run_layers_fused(pm355_model * m, const float * cur, float * d_x_out, const 
 }
 
 // x_in -> x_out for layers [lo, hi); positions from device memory d_pos (pos of token 0)
-int run_window(pm355_model * m, const int32_t * d_tokens, const float * d_x_in, int T, float * d_x_out,
+int run_window(pm_window * m, const int32_t * d_tokens, const float * d_x_in, int T, float * d_x_out,
                float * d_logits, int32_t * d_argmax, hipStream_t st) {
     (void) hipGetLastError();
     const pm355_hparams & hp = m->hp;
@@ -601,7 +627,7 @@ int run_window(pm355_model * m, const int32_t * d_tokens, const float * d_x_in, 
         m->flash_cells = attn_regime(m); m->long_ctx = m->flash_cells != 0;
         // ---- single token: every activation transform is fused into a mat-vec prologue / epilogue, 5 launches per layer
         const float * end = nullptr;
-        pm355_model::EnginePlan * eng = nullptr;
+        pm_window::EnginePlan * eng = nullptr;
         if (engine_eligible(m)) {
             hipStreamCaptureStatus cst = hipStreamCaptureStatusNone;
             const bool capturing = hipStreamIsCapturing(st, &cst) == hipSuccess && cst == hipStreamCaptureStatusActive;
@@ -866,15 +892,12 @@ int run_window(pm355_model * m, const int32_t * d_tokens, const float * d_x_in, 
 
 } // namespace
 
-extern "C" {
-
-pm355_model * pm355_model_new(const pm355_hparams * hp, int lo, int hi, int flags) {
+static pm355_model * window_new(const pm355_hparams * hp, int lo, int hi, int flags) {
     if (!hp || lo < 0 || hi > hp->n_layer || lo > hi) return nullptr;
     if (hp->head_dim % 8 || hp->n_embd % 256 || hp->n_head % hp->n_head_kv) return nullptr;
-    pm355_model * m = new pm355_model();
+    pm_window * m = new pm_window();
     m->hp = *hp; m->lo = lo; m->hi = hi; m->flags = flags;
     m->layers.resize(hi - lo);
-    m->err[0] = 0;
     m->rope.n_dims = hp->head_dim; m->rope.mode = hp->arch == 1 ? 2 : 0; m->rope.n_ctx_orig = hp->n_ctx_orig;
     m->rope.freq_base = hp->rope_freq_base; m->rope.freq_scale = hp->rope_freq_scale;
     m->rope.ext_factor = 0.0f; m->rope.attn_factor = 1.0f; m->rope.beta_fast = 32.0f; m->rope.beta_slow = 1.0f;
@@ -894,8 +917,8 @@ pm355_model * pm355_model_new(const pm355_hparams * hp, int lo, int hi, int flag
     return m;
 }
 
-void pm355_model_free(pm355_model * m) {
-    if (!m) return;
+pm_window::~pm_window() {
+    pm_window * m = this;
     (void) hipDeviceSynchronize();
     for (auto & g : m->graphs) (void) hipGraphExecDestroy(g.exec);
 #if PM_EXPERIMENTS
@@ -907,16 +930,15 @@ void pm355_model_free(pm355_model * m) {
     for (auto & L : m->layers) { for (auto & t : L.t) if (t.d) (void) hipFree(t.d); if (L.kc) (void) hipFree(L.kc); if (L.vc) (void) hipFree(L.vc); }
     Tensor * g[4] = {&m->tok_embd, &m->out_norm, &m->output, &m->rope_freqs};
     for (auto t : g) if (t->d) (void) hipFree(t->d);
-    void * s[] = {m->x, m->x1, m->q, m->k, m->v, m->att, m->h, m->h2, m->logits, m->xn, m->aq_k, m->aq_0, m->d_pos, m->d_tok, m->d_ctl, m->split_scratch, m->rope_tab, m->tab_big, m->ss, m->att_tk};
+    void * s[] = {m->x, m->x1, m->q, m->k, m->v, m->att, m->h, m->h2, m->logits, m->xn, m->aq_k, m->aq_0, m->d_pos, m->d_tok, m->d_ctl, m->split_scratch, m->rope_tab, m->tab_big, m->ss, m->att_tk, m->d_last, m->rows};
     for (auto p : s) if (p) (void) hipFree(p);
     pm355_uploader_free(m->up);
     if (m->cap_stream) (void) hipStreamDestroy(m->cap_stream);
     if (m->side) { (void) hipStreamDestroy(m->side); (void) hipEventDestroy(m->side_a); (void) hipEventDestroy(m->side_b); }
-    delete m;
 }
 
 // streaming mode: a freshly uploaded (and repacked) layer tensor is moved to pinned host memory; its device copy is released
-static int stream_park(pm355_model * m, int kind, int layer) {
+static int stream_park(pm_window * m, int kind, int layer) {
     if (!m->n_slots || kind >= 12) return 0;
     Layer & L = m->layers[layer - m->lo];
     Tensor & t = L.t[kind];
@@ -933,16 +955,17 @@ static int stream_park(pm355_model * m, int kind, int layer) {
     return 0;
 }
 
-int pm355_model_set_streaming(pm355_model * m, int n_slots) {
-    if (!m || m->finalized) return m ? seterr(m, PM355_E_SHAPE, "set_streaming: call before finalize") : PM355_E_SHAPE;
+int pm_window::set_streaming(int n) {
+    pm_window * m = this;
+    if (m->finalized) return seterr(m, PM355_E_SHAPE, "set_streaming: call before finalize");
     for (auto & L : m->layers) for (auto & t : L.t) if (t.d) return seterr(m, PM355_E_SHAPE, "set_streaming: call before the first layer tensor is set");
-    if (n_slots < 0 || n_slots > 1024) return seterr(m, PM355_E_RANGE, "set_streaming: n_slots");
-    m->n_slots = n_slots;
+    if (n < 0 || n > 1024) return seterr(m, PM355_E_RANGE, "set_streaming: n_slots");
+    m->n_slots = n;
     return 0;
 }
-uint64_t pm355_model_streamed_bytes(const pm355_model * m) { return m ? m->streamed_bytes : 0; }
 
-int pm355_model_set_tensor(pm355_model * m, int kind, int layer, int type, const void * host, size_t nbytes) {
+int pm_window::set_tensor(int kind, int layer, int type, const void * host, size_t nbytes) {
+    pm_window * m = this;
     (void) hipGetLastError();
     Tensor * t = tensor_slot(m, kind, layer);
     if (!t) return seterr(m, PM355_E_RANGE, "set_tensor: tensor not in this window");
@@ -957,7 +980,8 @@ int pm355_model_set_tensor(pm355_model * m, int kind, int layer, int type, const
     return stream_park(m, kind, layer);
 }
 
-int pm355_model_fill_tensor(pm355_model * m, int kind, int layer, int type, uint64_t seed, float scale) {
+int pm_window::fill_tensor(int kind, int layer, int type, uint64_t seed, float scale) {
+    pm_window * m = this;
     (void) hipGetLastError();
     Tensor * t = tensor_slot(m, kind, layer);
     if (!t) return seterr(m, PM355_E_RANGE, "fill_tensor: tensor not in this window");
@@ -975,12 +999,11 @@ int pm355_model_fill_tensor(pm355_model * m, int kind, int layer, int type, uint
     return stream_park(m, kind, layer);
 }
 
-int pm355_model_finalize(pm355_model * m, int max_tokens) { return pm355_model_finalize_seqs(m, max_tokens, 1); }
-
-int pm355_model_finalize_seqs(pm355_model * m, int max_tokens, int n_seq) {
+int pm_window::finalize(int max_tokens_, int n_seq_) {
+    pm_window * m = this;
     (void) hipGetLastError();
-    if (n_seq < 1 || n_seq > 64) return seterr(m, PM355_E_RANGE, "finalize: n_seq must be 1..64");
-    m->n_seq = n_seq;
+    if (n_seq_ < 1 || n_seq_ > 64) return seterr(m, PM355_E_RANGE, "finalize: n_seq must be 1..64");
+    m->n_seq = n_seq_;
     (void) pm355_uploader_sync(m->up);
     (void) hipDeviceSynchronize();
     // (a re-finalize re-allocates the KV caches, the rope table and the split scratch that the kept engine plans and captured graphs have baked in)
@@ -992,7 +1015,7 @@ int pm355_model_finalize_seqs(pm355_model * m, int max_tokens, int n_seq) {
     m->graphs.clear();
     const pm355_hparams & hp = m->hp;
     const size_t E = hp.n_embd, Eq = (size_t) hp.head_dim * hp.n_head, Ekv = (size_t) hp.head_dim * hp.n_head_kv, F = hp.n_ff;
-    const size_t T = max_tokens < 1 ? 1 : max_tokens;
+    const size_t T = max_tokens_ < 1 ? 1 : max_tokens_;
     m->max_tokens = (int) T;
     for (int il = m->lo; il < m->hi; ++il) {
         Layer & L = m->layers[il - m->lo];
@@ -1012,7 +1035,7 @@ int pm355_model_finalize_seqs(pm355_model * m, int max_tokens, int n_seq) {
               A((void **) &m->d_pos, 64 * 4) && A((void **) &m->d_ctl, 64) && A((void **) &m->d_tok, 64 + T * 4) &&
               A((void **) &m->rope_tab, (size_t) hp.head_dim * 4 * 32) &&      // cos / sin tables of up to 32 tokens (small-batch epilogue)
               A((void **) &m->ss, 2 * 256 * sizeof(double)) &&
-              A((void **) &m->att_tk, 65 * 4);
+              A((void **) &m->att_tk, 65 * 4) && A((void **) &m->d_last, 64 * 4);
     if (ok) (void) hipMemset(m->att_tk, 0, 65 * 4);
     if (ok && T > MMQ_MAX_TOKENS && !m->no_big) ok = A((void **) &m->tab_big, pm_mmq_big_table_bytes((int) ((maxK + 255) / 256 * 256), (int) T));
     if (!ok) return seterr(m, PM355_E_NOMEM, "finalize: scratch");
@@ -1035,7 +1058,7 @@ int pm355_model_finalize_seqs(pm355_model * m, int max_tokens, int n_seq) {
         for (int i = 0; i < m->n_slots; ++i) stream_prefetch(m, m->lo + i, i);
         m->stream_step = 0;
     }
-    m->h_pos.assign(n_seq, 0); m->h_seq = 0;
+    m->h_pos.assign(n_seq, 0); m->seq_open.assign(n_seq, 0); m->h_seq = 0;
     { const char * e = getenv("PM355_ATTN_SPLIT_MIN"); if (e && e[0]) m->split_min = atoi(e); }
     { const char * e = getenv("PM355_ATTN_FLASH"); m->use_flash = !(e && e[0] == '0'); }
     { const char * e = getenv("PM355_ATTN_MFMA"); m->attn_mfma = !(e && e[0] == '0'); }
@@ -1046,39 +1069,39 @@ int pm355_model_finalize_seqs(pm355_model * m, int max_tokens, int n_seq) {
     return hip_ok() ? 0 : seterr(m, PM355_E_HIP, "finalize");
 }
 
-size_t pm355_model_weight_bytes(const pm355_model * m) {
+size_t pm_window::weight_bytes() const {
+    const pm_window * m = this;
     size_t n = 0;
     for (auto & L : m->layers) for (int kd = 0; kd < 12; ++kd) n += L.t[kd].bytes;
     if (m->flags & PM355_HAS_HEAD) n += m->output.bytes + m->out_norm.bytes;
     return n;
 }
-size_t pm355_model_kv_bytes_per_pos(const pm355_model * m) {
+size_t pm_window::kv_bytes_per_pos() const {
+    const pm_window * m = this;
     return (size_t) (m->hi - m->lo) * 2 * (size_t) m->hp.head_dim * m->hp.n_head_kv * 2;
 }
-int pm355_model_kv_clear(pm355_model * m, pm355_stream_t st) {
+int pm_window::kv_clear(hipStream_t st) {
+    pm_window * m = this;
     const size_t kvb = (size_t) m->hp.head_dim * m->hp.n_head_kv * (size_t) m->hp.n_ctx * 2 * (size_t) m->n_seq;
     for (auto & L : m->layers) { (void) hipMemsetAsync(L.kc, 0, kvb, (hipStream_t) st); (void) hipMemsetAsync(L.vc, 0, kvb, (hipStream_t) st); }
     return 0;
 }
-void * pm355_model_kv_ptr(pm355_model * m, int layer, int which) {
+void * pm_window::kv_ptr(int layer, int which) {
+    pm_window * m = this;
     if (layer < m->lo || layer >= m->hi) return nullptr;
     return which ? m->layers[layer - m->lo].vc : m->layers[layer - m->lo].kc;
 }
-const char * pm355_model_error(pm355_model * m) { return m->err; }
-void * pm355_model_tensor_ptr(pm355_model * m, int kind, int layer, int * type_out) {
+void * pm_window::tensor_ptr(int kind, int layer, int * type_out) {
+    pm_window * m = this;
     Tensor * t = tensor_slot(m, kind, layer);
     if (!t || !t->d) return nullptr;
     if (type_out) *type_out = t->type;
     return t->d;
 }
 
-int pm355_model_set_pos(pm355_model * m, int pos, pm355_stream_t st) {
-    if (!m->finalized) return seterr(m, PM355_E_SHAPE, "set_pos: model not finalized");
-    return pm355_model_set_seq_pos(m, -1, pos, st);
-}
-
 // seq >= 0: set that sequence's position (does not change the current sequence); seq == -1: sequence 0 and make it current
-int pm355_model_set_seq_pos(pm355_model * m, int seq, int pos, pm355_stream_t st) {
+int pm_window::set_seq_pos(int seq, int pos, hipStream_t st) {
+    pm_window * m = this;
     if (!m->finalized) return seterr(m, PM355_E_SHAPE, "set_seq_pos: model not finalized");
     if (seq >= m->n_seq) return seterr(m, PM355_E_RANGE, "set_seq_pos: seq >= n_seq");
     if (pos < 0 || pos > m->hp.n_ctx) return seterr(m, PM355_E_RANGE, "set_seq_pos: position outside [0, n_ctx]");
@@ -1088,13 +1111,15 @@ int pm355_model_set_seq_pos(pm355_model * m, int seq, int pos, pm355_stream_t st
     m->h_pos[seq] = pos;
     return 0;
 }
-int pm355_model_set_seq(pm355_model * m, int seq, pm355_stream_t st) {
+int pm_window::set_seq(int seq, hipStream_t st) {
+    pm_window * m = this;
     if (!m->finalized || seq < 0 || seq >= m->n_seq) return seterr(m, PM355_E_RANGE, "set_seq: bad sequence id");
     pm_launch_set_i32(m->d_ctl, seq, (hipStream_t) st);
     m->h_seq = seq;
     return 0;
 }
-int pm355_model_head(pm355_model * m, const float * d_x_row, float * d_logits, int32_t * d_argmax, pm355_stream_t st) {
+int pm_window::head(const float * d_x_row, float * d_logits, int32_t * d_argmax, hipStream_t st) {
+    pm_window * m = this;
     if (!m->finalized || !(m->flags & PM355_HAS_HEAD)) return seterr(m, PM355_E_UNSUPPORTED, "head: window has no head");
     (void) hipGetLastError();
     int rc = run_head(m, d_x_row, d_logits, d_argmax, (hipStream_t) st);
@@ -1102,35 +1127,22 @@ int pm355_model_head(pm355_model * m, const float * d_x_row, float * d_logits, i
     return hip_ok() ? 0 : seterr(m, PM355_E_HIP, "head: kernel launch failed");
 }
 
-int pm355_model_decode(pm355_model * m, const int32_t * d_tokens, const float * d_x_in, int T, int pos0,
-                       float * d_x_out, float * d_logits, int32_t * d_argmax, pm355_stream_t st) {
+// one portion of one sequence (seq < 0: sequence 0, made current; the device counter and its mirror stay at pos0; else `seq` stays current)
+int pm_window::decode(int seq, const int32_t * d_tokens, const float * d_x_in, int T, int pos0, float * d_x_out, float * d_logits, int32_t * d_argmax, hipStream_t st) {
+    pm_window * m = this;
     if (!m->finalized) return seterr(m, PM355_E_SHAPE, "decode: model not finalized");
     if (T < 1 || T > m->max_tokens) return seterr(m, PM355_E_RANGE, "decode: n_tokens exceeds finalize(max_tokens)");
     if (pos0 < 0 || pos0 + T > m->hp.n_ctx) return seterr(m, PM355_E_RANGE, "decode: position outside n_ctx");
-    int rc = pm355_model_set_pos(m, pos0, st);
+    int rc = set_seq_pos(seq, pos0, st);
+    if (!rc && seq >= 0) rc = set_seq(seq, st);
     if (rc) return rc;
-    return run_window(m, d_tokens, d_x_in, T, d_x_out, d_logits, d_argmax, (hipStream_t) st);   // device counter and mirror stay at pos0
+    return run_window(m, d_tokens, d_x_in, T, d_x_out, d_logits, d_argmax, st);
 }
-
-// the same for sequence `seq` of a window finalized with n_seq > 1 (its KV slab, its position counter); leaves `seq` current
-int pm355_model_decode_seq(pm355_model * m, int seq, const int32_t * d_tokens, const float * d_x_in, int T, int pos0,
-                           float * d_x_out, float * d_logits, int32_t * d_argmax, pm355_stream_t st) {
-    if (!m->finalized) return seterr(m, PM355_E_SHAPE, "decode: model not finalized");
-    if (seq < 0 || seq >= m->n_seq) return seterr(m, PM355_E_RANGE, "decode_seq: seq >= n_seq");
-    if (T < 1 || T > m->max_tokens) return seterr(m, PM355_E_RANGE, "decode: n_tokens exceeds finalize(max_tokens)");
-    if (pos0 < 0 || pos0 + T > m->hp.n_ctx) return seterr(m, PM355_E_RANGE, "decode: position outside n_ctx");
-    int rc = pm355_model_set_seq_pos(m, seq, pos0, st);
-    if (!rc) rc = pm355_model_set_seq(m, seq, st);
-    if (rc) return rc;
-    return run_window(m, d_tokens, d_x_in, T, d_x_out, d_logits, d_argmax, (hipStream_t) st);
-}
-int pm355_model_n_embd(const pm355_model * m) { return m ? m->hp.n_embd : 0; }
-int pm355_model_n_seq(const pm355_model * m) { return m ? m->n_seq : 0; }
-int pm355_small_batch_max_tokens(void) { return MMQ_MAX_TOKENS; }
+extern "C" int pm355_small_batch_max_tokens(void) { return MMQ_MAX_TOKENS; }
 
 // head_first != 0 (ring rank 0): d_x_in is the LAST rank's activation; apply the head to it (-> d_argmax / d_logits),
 // then embed the token found at d_token (which may be d_argmax itself) and run the window -> d_x_out.
-static int step_body(pm355_model * m, const int32_t * d_token, const float * d_x_in, float * d_x_out,
+static int step_body(pm_window * m, const int32_t * d_token, const float * d_x_in, float * d_x_out,
                      float * d_logits, int32_t * d_argmax, int advance, int rotate, int head_first, hipStream_t st) {
     int rc;
     if (head_first) {
@@ -1146,14 +1158,10 @@ static int step_body(pm355_model * m, const int32_t * d_token, const float * d_x
     return 0;
 }
 
-int pm355_model_step(pm355_model * m, const int32_t * d_token, const float * d_x_in, float * d_x_out,
-                     float * d_logits, int32_t * d_argmax, int advance, int use_graph, pm355_stream_t pst) {
-    return pm355_model_step_ex(m, d_token, d_x_in, d_x_out, d_logits, d_argmax, advance, 0, 0, use_graph, pst);
-}
-
-int pm355_model_step_ex(pm355_model * m, const int32_t * d_token, const float * d_x_in, float * d_x_out,
-                        float * d_logits, int32_t * d_argmax, int advance, int rotate, int head_first, int use_graph,
-                        pm355_stream_t pst) {
+int pm_window::step_ex(const int32_t * d_token, const float * d_x_in, float * d_x_out,
+                       float * d_logits, int32_t * d_argmax, int advance, int rotate, int head_first, int use_graph,
+                       hipStream_t pst) {
+    pm_window * m = this;
     if (!m->finalized) return seterr(m, PM355_E_SHAPE, "step: model not finalized");
     if (head_first && (!(m->flags & PM355_HAS_HEAD) || !d_token || !d_x_in)) return seterr(m, PM355_E_SHAPE, "step: head_first needs HEAD, d_token and d_x_in");
     hipStream_t st = (hipStream_t) pst;
@@ -1199,8 +1207,8 @@ int pm355_model_step_ex(pm355_model * m, const int32_t * d_token, const float * 
 }
 
 // Synchronizes the device; non-zero if the window's launches left an error behind.
-int pm355_model_check(pm355_model * m) {
-    if (!m) return PM355_E_SHAPE;
+int pm_window::check() {
+    pm_window * m = this;
     if (hipDeviceSynchronize() != hipSuccess) return seterr(m, PM355_E_HIP, "check: device error");
     if (m->att_tk) {
         int w = 0;
@@ -1221,20 +1229,84 @@ int pm355_model_check(pm355_model * m) {
 
 // d_tokens_io[i] -> d_tokens_io[i+1]: the per-step graph reads its token from m->d_tok[0] and writes argmax to
 // m->d_tok[1]; two tiny D2D copies per step move tokens in and out (all on the stream, no host sync).
-int pm355_model_generate(pm355_model * m, int32_t * d_io, int pos0, int n_steps, int use_graph, pm355_stream_t pst) {
+int pm_window::generate(int32_t * d_io, int pos0, int n_steps, int use_graph, hipStream_t pst) {
+    pm_window * m = this;
     if (!m->finalized) return seterr(m, PM355_E_SHAPE, "generate: model not finalized");
     if (!(m->flags & PM355_HAS_EMBD) || !(m->flags & PM355_HAS_HEAD)) return seterr(m, PM355_E_UNSUPPORTED, "generate: needs EMBD and HEAD");
     if (pos0 < 0 || pos0 + n_steps > m->hp.n_ctx) return seterr(m, PM355_E_RANGE, "generate: position outside n_ctx");
     hipStream_t st = (hipStream_t) pst;
-    int rc = pm355_model_set_pos(m, pos0, pst);
+    int rc = set_seq_pos(-1, pos0, pst);
     if (rc) return rc;
     for (int i = 0; i < n_steps; ++i) {
         (void) hipMemcpyAsync(m->d_tok, d_io + i, 4, hipMemcpyDeviceToDevice, st);
-        rc = pm355_model_step(m, m->d_tok, nullptr, nullptr, nullptr, m->d_tok + 1, 1, use_graph, pst);
+        rc = step_ex(m->d_tok, nullptr, nullptr, nullptr, m->d_tok + 1, 1, 0, 0, use_graph, pst);
         if (rc) return rc;
         (void) hipMemcpyAsync(d_io + i + 1, m->d_tok + 1, 4, hipMemcpyDeviceToDevice, st);
     }
     return 0;
 }
 
-} // extern "C"
+// ---- batches: every entry is a portion of one open sequence; a sequence holds one KV slab of n_ctx cells, portions run one after another ----------------------
+int pm_window::finalize_pool(int max_tokens_, int n_seq_, int64_t pool_tokens) {
+    if (pool_tokens > (int64_t) n_seq_ * hp.n_ctx) return seterr(this, PM355_E_RANGE, "finalize_pool: more tokens than n_seq slabs of n_ctx cells hold");
+    if (!(flags & PM355_HAS_EMBD) || !(flags & PM355_HAS_HEAD)) return seterr(this, PM355_E_UNSUPPORTED, "finalize_pool: batches need the embedding and the head");
+    const int rc = finalize(max_tokens_, n_seq_);
+    if (rc) return rc;
+    return hipMalloc((void **) &rows, (size_t) max_tokens * hp.n_embd * 4 + 256) == hipSuccess ? 0 : seterr(this, PM355_E_NOMEM, "finalize_pool: hidden rows");
+}
+int pm_window::seq_new() {
+    if (!finalized) return seterr(this, PM355_E_SHAPE, "seq_new: model not finalized");
+    for (int s = 0; s < n_seq; ++s) if (!seq_open[s]) { seq_open[s] = 1; h_pos[s] = 0; return s; }
+    return seterr(this, PM355_E_NOMEM, "seq_new: every KV slab is taken");
+}
+int pm_window::seq_free(int seq) {
+    if (seq < 0 || seq >= n_seq || !seq_open[seq]) return seterr(this, PM355_E_RANGE, "seq_free: not an open sequence");
+    seq_open[seq] = 0; h_pos[seq] = 0;
+    return 0;
+}
+int pm_window::seq_len(int seq) { return (seq < 0 || seq >= n_seq || !seq_open[seq]) ? PM355_E_RANGE : h_pos[seq]; }
+int pm_window::pool_info(pm355_pool_info * o) {
+    *o = pm355_pool_info{hp.n_ctx, n_seq, 0, n_seq, 0, hp.n_ctx};
+    for (char c : seq_open) if (!c) { ++o->free_pages; ++o->free_seqs; }
+    return 0;
+}
+int pm_window::batch(const pm355_batch_entry * e, int n, float * d_logits, int32_t * d_argmax, hipStream_t st) {
+    pm_window * m = this;
+    if (!finalized || !rows) return seterr(m, PM355_E_SHAPE, "batch: finalize_pool first");
+    for (int i = 0; i < n; ++i) {
+        if (e[i].seq < 0 || e[i].seq >= n_seq || !seq_open[e[i].seq] || e[i].n_tokens < 1) return seterr(m, PM355_E_RANGE, "batch: not an open sequence / no tokens");
+        if (!e[i].tokens && e[i].n_tokens != 1) return seterr(m, PM355_E_SHAPE, "batch: the device-side token is one token");
+        if (h_pos[e[i].seq] + e[i].n_tokens > hp.n_ctx) return seterr(m, PM355_E_NOMEM, "batch: the sequence would outgrow its KV slab");
+        for (int j = 0; j < i; ++j) if (e[j].seq == e[i].seq) return seterr(m, PM355_E_SHAPE, "batch: a sequence appears twice");
+        for (int j = 0; j < e[i].n_want; ++j) if (e[i].want[j] < 0 || e[i].want[j] >= e[i].n_tokens) return seterr(m, PM355_E_RANGE, "batch: want outside the portion");
+        for (int j = 0; e[i].tokens && j < e[i].n_tokens; ++j) if (e[i].tokens[j] < 0 || e[i].tokens[j] >= hp.n_vocab) return seterr(m, PM355_E_RANGE, "batch: token id outside the vocabulary");
+    }
+    size_t row = 0;
+    for (int i = 0; i < n; ++i) {
+        const int seq = e[i].seq;
+        for (int off = 0; off < e[i].n_tokens; off += max_tokens) {
+            const int T = std::min(max_tokens, e[i].n_tokens - off), pos = h_pos[seq];
+            bool want = false;
+            for (int j = 0; j < e[i].n_want; ++j) want = want || (e[i].want[j] >= off && e[i].want[j] < off + T);
+            if (e[i].tokens && hipMemcpyAsync(d_tok, e[i].tokens + off, (size_t) T * 4, hipMemcpyHostToDevice, st) != hipSuccess) return seterr(m, PM355_E_HIP, "batch: token upload");
+            if (!e[i].tokens && hipMemcpyAsync(d_tok, d_last + seq, 4, hipMemcpyDeviceToDevice, st) != hipSuccess) return seterr(m, PM355_E_HIP, "batch: token copy");
+            int rc = decode(seq, d_tok, nullptr, T, pos, want ? rows : nullptr, nullptr, nullptr, st);
+            if (rc) return rc;
+            for (int j = 0; j < e[i].n_want; ++j) {
+                const int w = e[i].want[j] - off;
+                if (w < 0 || w >= T) continue;
+                // (rows are counted in the order of `want`, which need not be ascending)
+                float * lg = d_logits ? d_logits + (row + j) * hp.n_vocab : nullptr;
+                rc = run_head(m, rows + (size_t) w * hp.n_embd, lg, d_argmax ? d_argmax + row + j : nullptr, st);
+                if (rc) return rc;
+                if (d_argmax && j == e[i].n_want - 1) (void) hipMemcpyAsync(d_last + seq, d_argmax + row + j, 4, hipMemcpyDeviceToDevice, st);
+            }
+            rc = set_seq_pos(seq, pos + T, st);
+            if (rc) return rc;
+        }
+        row += e[i].n_want;
+    }
+    return hip_ok() ? 0 : seterr(m, PM355_E_HIP, "batch: kernel launch failed");
+}
+
+static const pm_arch_registrar reg_llama({0, "llama", window_new, nullptr}), reg_qwen2({1, "qwen2", window_new, nullptr});

@@ -145,26 +145,6 @@ static int num_cus() {
 
 int pm_gemv_units_per_row(int type, int64_t K) { return (int) (K / nv_of(type)); }
 
-size_t pm_weight_row_bytes(int type, int64_t K) {
-    switch (type) {
-        case PM_F32:  return (size_t) K * 4;
-        case PM_F16:  return (size_t) K * 2;
-        case PM_Q8_0: return (size_t) (K / 32) * PM_BS_Q8_0;
-        case PM_Q4_K: return (size_t) (K / 256) * PM_BS_Q4_K;
-        case PM_Q5_K: return (size_t) (K / 256) * PM_BS_Q5_K;
-        case PM_Q6_K: return (size_t) (K / 256) * PM_BS_Q6_K;
-    }
-    return 0;
-}
-
-size_t pm_weight_row_stride(int type, int64_t K) {
-    switch (type) {
-        case PM_Q8_0: { const size_t nb = K / 32;  return nb * 32 + ((nb * 2 + 15) & ~(size_t) 15); }
-        case PM_Q6_K: return pm_q6k_row_stride((size_t) (K / 256));
-    }
-    return pm_weight_row_bytes(type, K);
-}
-
 // Validates a fused job list and fills the kernel argument block. ta <= tb are the (at most two) quant types in the
 // canonical order of the instantiated kernels: (Q4_K,Q4_K) (Q5_K,Q5_K) (Q6_K,Q6_K) (Q8_0,Q8_0) (Q4_K,Q6_K) (Q4_K,Q5_K); job 0 is
 // always a `ta` job (the kernel pre-issues it). grid_fixed > 0: the caller's grid (attn_wo.hip), else chosen here.

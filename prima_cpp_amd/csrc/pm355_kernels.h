@@ -27,6 +27,8 @@ static inline void pm_allow_big_lds(const void * kern, size_t lds) {
     if (n_done < 256) { done[n_done].k = kern; done[n_done].dev = dev; ++n_done; }
 }
 
+int pm_api_fail(int code, const char * what, hipError_t e);      // sets pm355_last_error(), returns code (c_api_base.hip)
+
 // bytes of one quantized ACTIVATION row in the library's internal row-SoA layout (quantize.hip)
 static inline size_t pm_q8k_row_bytes(int K) { return (size_t) K + (size_t) (K / 256) * 4 + (size_t) (K / 16) * 2; }
 static inline size_t pm_q80_row_bytes(int K) { return (size_t) K + (size_t) (K / 32) * 2; }

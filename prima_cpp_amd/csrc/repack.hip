@@ -52,6 +52,26 @@ __global__ __launch_bounds__(256) void repack_kernel(const uint16_t * __restrict
     else           dst[row * row_halfs + o / 2] = src[row * stride_halfs + so / 2];
 }
 
+size_t pm_weight_row_bytes(int type, int64_t K) {
+    switch (type) {
+        case PM_F32:  return (size_t) K * 4;
+        case PM_F16:  return (size_t) K * 2;
+        case PM_Q8_0: return (size_t) (K / 32) * PM_BS_Q8_0;
+        case PM_Q4_K: return (size_t) (K / 256) * PM_BS_Q4_K;
+        case PM_Q5_K: return (size_t) (K / 256) * PM_BS_Q5_K;
+        case PM_Q6_K: return (size_t) (K / 256) * PM_BS_Q6_K;
+    }
+    return 0;
+}
+
+size_t pm_weight_row_stride(int type, int64_t K) {
+    switch (type) {
+        case PM_Q8_0: { const size_t nb = K / 32;  return nb * 32 + ((nb * 2 + 15) & ~(size_t) 15); }
+        case PM_Q6_K: return pm_q6k_row_stride((size_t) (K / 256));
+    }
+    return pm_weight_row_bytes(type, K);
+}
+
 void pm_launch_repack(int type, const void * src, void * dst, int64_t K, int64_t nrows, int to_device, hipStream_t st) {
     const size_t rb = pm_weight_row_bytes(type, K);
     if (!pm_type_is_repacked(type)) {

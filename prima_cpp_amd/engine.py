@@ -7,10 +7,11 @@ import numpy as np
 import torch
 
 from . import lib as L
-from .lib import F32, Q4_K, Q5_K, Q6_K, Q8_0, check, ptr, stream_ptr  # noqa: F401
+from .lib import BF16, F32, Q4_K, Q5_K, Q6_K, Q8_0, check, ptr, stream_ptr  # noqa: F401
 
 (T_ATTN_NORM, T_WQ, T_WK, T_WV, T_WO, T_FFN_NORM, T_FFN_GATE, T_FFN_UP, T_FFN_DOWN, T_BQ, T_BK, T_BV,
- T_TOK_EMBD, T_OUT_NORM, T_OUTPUT, T_ROPE_FREQS) = range(16)
+ T_TOK_EMBD, T_OUT_NORM, T_OUTPUT, T_ROPE_FREQS, T_ATTN_NORM_B, T_FFN_NORM_B, T_OUT_NORM_B, T_W_OUT_GATE, T_SINK, T_VALUE_MIX, T_FFN_UP_B,
+ T_FFN_DOWN_B) = range(24)
 HAS_EMBD, HAS_HEAD = 1, 2
 
 _vp, _i32, _i64, _sz = C.c_void_p, C.c_int, C.c_int64, C.c_size_t
@@ -22,6 +23,32 @@ class HParams(C.Structure):
                 ("n_ctx", C.c_int32), ("n_ctx_orig", C.c_int32),
                 ("rms_eps", C.c_float), ("rope_freq_base", C.c_float), ("rope_freq_scale", C.c_float),
                 ("pad_", C.c_int32)]
+
+
+class LayerSpec(C.Structure):
+    """One layer of a layer-described model (pm355_layer_spec): sizes, mechanisms, constants."""
+    _fields_ = [("n_head", C.c_int32), ("n_head_kv", C.c_int32), ("k_dim", C.c_int32), ("v_dim", C.c_int32),
+                ("mix_flags", C.c_int32), ("mask", C.c_int32), ("mask_size", C.c_int32), ("scale", C.c_float), ("softcap", C.c_float),
+                ("ff", C.c_int32), ("n_ff", C.c_int32), ("act", C.c_int32)]
+
+
+MIX_QK_NORM, MIX_SINK, MIX_VALUE_MIX, MIX_OUT_GATE = 1, 2, 4, 8
+MASK_CAUSAL, MASK_CHUNK = 0, 1
+FF_NONE, FF_DENSE = 0, 1
+ACT_NONE, ACT_RELU2 = 0, 1
+
+
+class StackDesc(C.Structure):
+    _fields_ = [("arch", C.c_int32), ("n_layer", C.c_int32), ("n_embd", C.c_int32), ("n_vocab", C.c_int32), ("type", C.c_int32),
+                ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec))]
+
+
+class BatchEntry(C.Structure):
+    _fields_ = [("seq", C.c_int32), ("n_tokens", C.c_int32), ("tokens", C.c_void_p), ("n_want", C.c_int32), ("want", C.c_void_p)]
+
+
+class PoolInfo(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("page_tokens", "n_pages", "free_pages", "n_seqs", "free_seqs", "max_seq_tokens")]
 
 
 LLAMA3_8B = dict(arch=0, n_layer=32, n_embd=4096, n_head=32, n_head_kv=8, head_dim=128, n_ff=14336, n_vocab=128256,
@@ -80,6 +107,15 @@ def _lib():
             "pm355_model_step": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _vp]),
             "pm355_model_set_streaming": (_i32, [_vp, _i32]),
             "pm355_model_streamed_bytes": (C.c_uint64, [_vp]),
+            "pm355_arch_id": (_i32, [C.c_char_p]),
+            "pm355_model_new_stack": (_vp, [C.POINTER(StackDesc)]),
+            "pm355_model_finalize_pool": (_i32, [_vp, _i32, _i32, _i64]),
+            "pm355_model_seq_new": (_i32, [_vp]),
+            "pm355_model_seq_free": (_i32, [_vp, _i32]),
+            "pm355_model_seq_len": (_i32, [_vp, _i32]),
+            "pm355_model_pool_info": (_i32, [_vp, C.POINTER(PoolInfo)]),
+            "pm355_model_batch": (_i32, [_vp, C.POINTER(BatchEntry), _i32, _vp, _vp, _vp]),
+            "pm355_model_n_vocab": (_i32, [_vp]),
         }
         for name, (res, args) in S.items():
             f = getattr(lib, name)
@@ -88,27 +124,15 @@ def _lib():
     return lib
 
 
-class Window:
-    """Layers [lo, hi) of a model resident on the current device (+ tok_embd / head when flagged)."""
+class Model:
+    """A pm355_model handle: what every architecture has (tensors, sequences, batches)."""
 
-    def __init__(self, hp, lo=0, hi=None, flags=HAS_EMBD | HAS_HEAD, n_ctx=512):
-        self.lib = _lib()
-        hp = dict(hp)
-        hp.setdefault("n_ctx_orig", 8192)
-        hp.setdefault("rope_freq_scale", 1.0)
-        hp["n_ctx"] = n_ctx
-        self.hp_dict = hp
-        self.hp = HParams(**{k: v for k, v in hp.items() if k in dict(HParams._fields_)})
-        self.lo, self.hi = lo, hp["n_layer"] if hi is None else hi
-        self.flags = flags
-        self.h = self.lib.pm355_model_new(C.byref(self.hp), self.lo, self.hi, flags)
-        if not self.h:
-            raise L.PM355Error("pm355_model_new failed (bad hparams / window)")
-        self.dev = torch.device("cuda", torch.cuda.current_device())
+    h = None
 
     def _chk(self, rc, what):
-        if rc != 0:
+        if rc < 0:
             raise L.PM355Error(f"{what}: rc={rc}: {self.lib.pm355_model_error(self.h).decode()}")
+        return rc
 
     def close(self):
         if self.h:
@@ -129,6 +153,64 @@ class Window:
 
     def fill_tensor(self, kind, layer, qtype, seed, scale):
         self._chk(self.lib.pm355_model_fill_tensor(self.h, kind, layer, qtype, seed, scale), "fill_tensor")
+
+    # ---- sequences and batches ---------------------------------------------------------------
+    def finalize_pool(self, max_tokens, n_seq, pool_tokens):
+        """Cache for n_seq open sequences with at most pool_tokens tokens together, scratch for max_tokens tokens per pass."""
+        self._chk(self.lib.pm355_model_finalize_pool(self.h, max_tokens, n_seq, pool_tokens), "finalize_pool")
+
+    @property
+    def n_vocab(self):
+        return self.lib.pm355_model_n_vocab(self.h)
+
+    def seq_new(self):
+        return self._chk(self.lib.pm355_model_seq_new(self.h), "seq_new")
+
+    def seq_free(self, seq):
+        self._chk(self.lib.pm355_model_seq_free(self.h, seq), "seq_free")
+
+    def seq_len(self, seq):
+        return self._chk(self.lib.pm355_model_seq_len(self.h, seq), "seq_len")
+
+    def pool_info(self):
+        p = PoolInfo()
+        self._chk(self.lib.pm355_model_pool_info(self.h, C.byref(p)), "pool_info")
+        return p
+
+    def batch(self, entries, logits=None, argmax=None):
+        """One step. entries: (seq, tokens or None, want) - None: the sequence's last greedy token, taken on the device. logits: f32 device tensor
+        [wanted rows, n_vocab]; argmax: int32 device tensor [wanted rows]; rows in the order of entries and of want."""
+        arr, keep = (BatchEntry * len(entries))(), []
+        for e, (seq, tokens, want) in zip(arr, entries):
+            w = np.asarray(want, dtype=np.int32)
+            t = None if tokens is None else np.ascontiguousarray(tokens, dtype=np.int32)
+            keep += [w, t]
+            e.seq, e.n_tokens, e.tokens = seq, 1 if t is None else t.size, None if t is None else t.ctypes.data
+            e.n_want, e.want = w.size, w.ctypes.data
+        rows = sum(e.n_want for e in arr)
+        for name, out, n in (("logits", logits, rows * self.n_vocab), ("argmax", argmax, rows)):
+            if out is not None and out.numel() < n:
+                raise L.PM355Error(f"batch: {name} is too small")
+        self._chk(self.lib.pm355_model_batch(self.h, arr, len(entries), ptr(logits), ptr(argmax), stream_ptr()), "batch")
+
+
+class Window(Model):
+    """Layers [lo, hi) of a model resident on the current device (+ tok_embd / head when flagged)."""
+
+    def __init__(self, hp, lo=0, hi=None, flags=HAS_EMBD | HAS_HEAD, n_ctx=512):
+        self.lib = _lib()
+        hp = dict(hp)
+        hp.setdefault("n_ctx_orig", 8192)
+        hp.setdefault("rope_freq_scale", 1.0)
+        hp["n_ctx"] = n_ctx
+        self.hp_dict = hp
+        self.hp = HParams(**{k: v for k, v in hp.items() if k in dict(HParams._fields_)})
+        self.lo, self.hi = lo, hp["n_layer"] if hi is None else hi
+        self.flags = flags
+        self.h = self.lib.pm355_model_new(C.byref(self.hp), self.lo, self.hi, flags)
+        if not self.h:
+            raise L.PM355Error("pm355_model_new failed (bad hparams / window, or an architecture this build does not carry)")
+        self.dev = torch.device("cuda", torch.cuda.current_device())
 
     def load_desc(self, desc):
         """Load from a tests/_bind.ModelDesc (host pointers, GGUF block order)."""
@@ -287,6 +369,50 @@ class Window:
     def step(self, token=None, x_in=None, x_out=None, logits=None, argmax=None, advance=1, use_graph=True):
         self._chk(self.lib.pm355_model_step(self.h, ptr(token), ptr(x_in), ptr(x_out), ptr(logits), ptr(argmax), advance,
                                             int(use_graph), stream_ptr()), "step")
+
+
+
+class Stack(Model):
+    """A layer-described model with dense weights and a paged cache (pm355_model_new_stack). layers: LayerSpec list; type BF16 or F32."""
+
+    def __init__(self, arch, layers, n_embd, n_vocab, norm_eps, type=BF16):
+        self.lib = _lib()
+        self.specs = (LayerSpec * len(layers))(*layers)
+        aid = self.lib.pm355_arch_id(arch.encode())
+        if aid < 0:
+            raise L.PM355Error(f"architecture {arch} is not in this build")
+        self.desc = StackDesc(aid, len(layers), n_embd, n_vocab, type, norm_eps, self.specs)
+        self.h = self.lib.pm355_model_new_stack(C.byref(self.desc))
+        if not self.h:
+            raise L.PM355Error("pm355_model_new_stack failed (sizes out of range, or not enough memory)")
+        self.type = type
+        self.dev = torch.device("cuda", torch.cuda.current_device())
+
+    @property
+    def weight_bytes(self):
+        return self.lib.pm355_model_weight_bytes(self.h)
+
+    @property
+    def kv_bytes_per_pos(self):
+        return self.lib.pm355_model_kv_bytes_per_pos(self.h)
+
+    def fill_synthetic(self, seed=1234):
+        """Random weights generated in HBM (bench)."""
+        E = self.desc.n_embd
+        self.fill_tensor(T_TOK_EMBD, -1, self.type, seed + 1, 1.0)
+        self.fill_tensor(T_OUTPUT, -1, self.type, seed + 2, 2.0 / np.sqrt(E))
+        self.fill_tensor(T_OUT_NORM, -1, F32, seed + 3, 0.0)
+        self.fill_tensor(T_OUT_NORM_B, -1, F32, seed + 4, 0.1)
+        for i, s in enumerate(self.specs):
+            k = seed * 1000003 + i * 131
+            for j, (kind, width) in enumerate(((T_WQ, E), (T_WK, E), (T_WV, E), (T_WO, s.n_head * s.v_dim), (T_W_OUT_GATE, E if s.mix_flags & MIX_OUT_GATE else 0),
+                                               (T_FFN_UP, E if s.ff else 0), (T_FFN_DOWN, s.n_ff if s.ff else 0))):
+                if width:
+                    self.fill_tensor(kind, i, self.type, k + j, 2.0 / np.sqrt(width))
+            for j, (kind, on) in enumerate(((T_ATTN_NORM, 1), (T_ATTN_NORM_B, 1), (T_FFN_NORM, s.ff), (T_FFN_NORM_B, s.ff), (T_FFN_UP_B, s.ff), (T_FFN_DOWN_B, s.ff),
+                                            (T_SINK, s.mix_flags & MIX_SINK), (T_VALUE_MIX, s.mix_flags & MIX_VALUE_MIX))):
+                if on:
+                    self.fill_tensor(kind, i, F32, k + 50 + j, 0.1)
 
 
 def smoke(oracle):

@@ -8,8 +8,8 @@ import os
 
 import torch  # noqa: F401  (must precede the CDLL below: shared HIP runtime)
 
-F32, F16, Q8_0, Q4_K, Q5_K, Q6_K, Q8_K = 0, 1, 8, 12, 13, 14, 15
-_BLOCK = {Q8_0: (32, 34), Q4_K: (256, 144), Q5_K: (256, 176), Q6_K: (256, 210), Q8_K: (256, 292), F16: (1, 2), F32: (1, 4)}
+F32, F16, Q8_0, Q4_K, Q5_K, Q6_K, Q8_K, BF16 = 0, 1, 8, 12, 13, 14, 15, 30
+_BLOCK = {Q8_0: (32, 34), Q4_K: (256, 144), Q5_K: (256, 176), Q6_K: (256, 210), Q8_K: (256, 292), F16: (1, 2), F32: (1, 4), BF16: (1, 2)}
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 
@@ -19,8 +19,12 @@ class PM355Error(RuntimeError):
 
 
 def lib_path():
-    """In-tree library; PM355_LIB selects another build of the same C ABI (A/B kernel experiments)."""
-    return os.environ.get("PM355_LIB") or os.path.join(HERE, "libprima_mi355.so")
+    """In-tree library; PM355_LIB selects another build of the same C ABI (A/B kernel experiments). Where only the dense-weight subset is built
+    (libprima_mi355_dense.so, build.build_dense()), that one: its architecture registry says what it serves."""
+    if os.environ.get("PM355_LIB"):
+        return os.environ["PM355_LIB"]
+    full, dense = os.path.join(HERE, "libprima_mi355.so"), os.path.join(HERE, "libprima_mi355_dense.so")
+    return dense if os.path.exists(dense) and not os.path.exists(full) else full
 
 
 _lib = None
