@@ -412,6 +412,35 @@ PM355_API int pm355_op_mul_mat_f(const pm355_tensor * a, const pm355_tensor * b,
 PM355_API int pm355_op_get_rows_f32(const pm355_tensor * a, const int32_t * d_idx, int64_t n_idx, const pm355_tensor * dst,
                                     pm355_stream_t stream);
 
+/* ---- (A") dense weights and paged caches (prima_cpp_amd/csrc/dense_*.hip, attn_paged.hip): what layer-described models run on ----------------
+ * type = PM355_TYPE_BF16 (bf16 operands, f32 accumulation) or PM355_TYPE_F32 (32-bit throughout). Matrices and activations are rows of K values, K a multiple of 64
+ * (zero padding), W has N rows, N a multiple of 64. */
+/* y[t][n] = act(W[n] . x[t] + bias[n]) for n < n_store; y: y_type, ldy values per token; act = PM355_ACT_* */
+PM355_API int pm355_dense_mul_mat(int type, const void * W, int64_t K, int64_t N, const void * x, int64_t ldx, int n_tokens, void * y, int64_t ldy, int y_type, int64_t n_store,
+                                  const float * bias, int act, pm355_stream_t stream);
+/* the same for x = r + layer_norm(d) (weight w, bias b, both f32 rows of `width` <= K values), formed inside the launch; the sum is also written to r_out (1..4 tokens) */
+PM355_API int pm355_dense_mul_mat_norm(int type, const void * W, int64_t K, int64_t N, const float * r, const float * d, int64_t ld, const float * w, const float * b, float eps,
+                                       int width, float * r_out, int n_tokens, void * y, int64_t ldy, int y_type, int64_t n_store, const float * bias, int act,
+                                       pm355_stream_t stream);
+/* r += layer_norm(d), xb = the sum in `type` (or NULL) */
+PM355_API int pm355_add_layer_norm(int type, float * r, const float * d, int64_t ld, const float * w, const float * b, float eps, int width, int n_rows, void * xb,
+                                   pm355_stream_t stream);
+/* One attention layer over paged caches (mechanisms: PM355_MIX_*, PM355_MASK_* below). Head sizes in caches and q rows are padded (k_pad, v_pad: multiples of 64; for the
+ * matrix-core kernels 64 / 128, or 256 both): k_pages [page][n_head_kv][64][k_pad], v_pages [page][n_head_kv][v_pad][64]. proj: f32 or bf16 rows
+ * [q | k | v | gate] of ld_proj values. mode: 0 = unit norms, value mixing and the cache store only; 1 = 0 and the vector-pipe attention; 2 = 0 and the prompt kernel
+ * over tiles of up to 128 tokens (int32 {row, tokens, position, sequence} each, device memory); 3 = decode kernel with 0's work inside, one token per row; +16: without
+ * 0's work (already done). */
+typedef struct {
+    int32_t type, n_head, n_head_kv, k_dim, v_dim, k_pad, v_pad, mix_flags, mask, mask_size; float scale, softcap, eps, lambda;
+    int32_t mixes;                        /* 1: v is mixed with v_first, 2: v becomes v_first */
+    const float * sink; void * k_pages; void * v_pages; float * v_first; int32_t ld_v_first;
+    const void * proj; int32_t ld_proj, proj_type; void * q; void * out; int32_t ldo;
+    const int32_t * d_pos; const int32_t * d_seq; const int32_t * d_table; int32_t table_ld, n_tokens, max_keys;
+    const int32_t * d_tiles; int32_t n_tiles; float * scratch; size_t scratch_floats; uint32_t * tickets;      /* split keys: pm355_attn_paged_scratch(); zeroed once */
+} pm355_attn_paged_args;
+PM355_API size_t pm355_attn_paged_scratch(int n_tokens, int n_head, int n_head_kv, int v_pad);      /* floats; tickets: n_tokens * n_head words */
+PM355_API int pm355_attn_paged(const pm355_attn_paged_args * a, int mode, pm355_stream_t stream);
+
 /* ---- (B) engine: resident decoder for one layer window --------------------------------------------- */
 typedef struct pm355_model pm355_model;
 

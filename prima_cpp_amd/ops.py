@@ -543,3 +543,52 @@ class EngineRun:
         lib.pm355_engine_run.argtypes = [C.c_void_p, C.c_int, C.c_void_p]
         arr = (EnginePhase * len(self.phases))(*self.phases)
         check(lib.pm355_engine_run(C.addressof(arr), len(self.phases), stream_ptr()), "engine_run")
+
+
+# ---- dense weights, paged caches (part A" of the C ABI) --------------------------------------------------------------------------
+_vp, _i32, _i64, _f32, _sz = L.C.c_void_p, L.C.c_int, L.C.c_int64, L.C.c_float, L.C.c_size_t
+
+
+class AttnPagedArgs(L.C.Structure):
+    _fields_ = ([(n, L.C.c_int32) for n in ("type", "n_head", "n_head_kv", "k_dim", "v_dim", "k_pad", "v_pad", "mix_flags", "mask", "mask_size")] +
+                [(n, _f32) for n in ("scale", "softcap", "eps", "lam")] + [("mixes", L.C.c_int32)] +
+                [(n, _vp) for n in ("sink", "k_pages", "v_pages", "v_first")] + [("ld_v_first", L.C.c_int32), ("proj", _vp), ("ld_proj", L.C.c_int32), ("proj_type", L.C.c_int32),
+                 ("q", _vp), ("out", _vp), ("ldo", L.C.c_int32)] + [(n, _vp) for n in ("d_pos", "d_seq", "d_table")] +
+                [(n, L.C.c_int32) for n in ("table_ld", "n_tokens", "max_keys")] + [("d_tiles", _vp), ("n_tiles", L.C.c_int32), ("scratch", _vp), ("scratch_floats", _sz), ("tickets", _vp)])
+
+
+def pm_type(t):
+    """pm355 type of a torch tensor"""
+    return {torch.float32: F32, torch.bfloat16: L.BF16}[t.dtype]
+
+
+def dense_mul_mat(w, x, y, n_store=None, bias=None, act=0):
+    """y[t, :n_store] = act(x @ w.T + bias); w [N, K], x [T, >= K] of one type (K, N multiples of 64), y f32 or bf16"""
+    f = L.declare("pm355_dense_mul_mat", _i32, [_i32, _vp, _i64, _i64, _vp, _i64, _i32, _vp, _i64, _i32, _i64, _vp, _i32, _vp])
+    check(f(pm_type(w), ptr(w), w.shape[1], w.shape[0], ptr(x), x.stride(0), x.shape[0], ptr(y), y.stride(0), pm_type(y), w.shape[0] if n_store is None else n_store, ptr(bias), act,
+            stream_ptr()), "dense_mul_mat")
+    return y
+
+
+def dense_mul_mat_norm(w, r, d, nw, nb, eps, r_out, y, width, bias=None, act=0):
+    """the same for x = r + layer_norm(d), which is also written to r_out (1..4 tokens)"""
+    f = L.declare("pm355_dense_mul_mat_norm", _i32, [_i32, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _vp, _f32, _i32, _vp, _i32, _vp, _i64, _i32, _i64, _vp, _i32, _vp])
+    check(f(pm_type(w), ptr(w), w.shape[1], w.shape[0], ptr(r), ptr(d), r.stride(0), ptr(nw), ptr(nb), eps, width, ptr(r_out), r.shape[0], ptr(y), y.stride(0), pm_type(y), y.shape[1],
+            ptr(bias), act, stream_ptr()), "dense_mul_mat_norm")
+    return y
+
+
+def add_layer_norm(r, d, nw, nb, eps, width, xb=None):
+    """r += layer_norm(d) in place; xb (bf16 or f32, like r) receives the sum"""
+    f = L.declare("pm355_add_layer_norm", _i32, [_i32, _vp, _vp, _i64, _vp, _vp, _f32, _i32, _i32, _vp, _vp])
+    check(f(F32 if xb is None else pm_type(xb), ptr(r), ptr(d), r.stride(0), ptr(nw), ptr(nb), eps, width, r.shape[0], ptr(xb), stream_ptr()), "add_layer_norm")
+
+
+def attn_paged(args, mode):
+    """one attention layer over paged caches (pm355_attn_paged): args = AttnPagedArgs of device pointers"""
+    f = L.declare("pm355_attn_paged", _i32, [L.C.POINTER(AttnPagedArgs), _i32, _vp])
+    check(f(L.C.byref(args), mode, stream_ptr()), "attn_paged")
+
+
+def attn_paged_scratch(n_tokens, n_head, n_head_kv, v_pad):
+    return L.declare("pm355_attn_paged_scratch", _sz, [_i32, _i32, _i32, _i32])(n_tokens, n_head, n_head_kv, v_pad)

@@ -46,11 +46,13 @@ def mix_values(v, first, lam):
 
 
 def attention(h, w, p, cfg, eps, first_values):
-    """returns (mixer output, first_values or this layer's own values where it is the first one that mixes)"""
+    """returns (mixer output, first_values or this layer's own values where it is the first one that mixes). The design has every mechanism; tests of one alone switch the
+    others off (unit_norm, has_sink, gate)."""
     n = h.shape[0]
     H, G, dk, dv = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
-    q = rms_unit((h @ w[p + "q"].T).reshape(n, H, dk), eps)
-    k = rms_unit((h @ w[p + "k"].T).reshape(n, G, dk), eps)
+    q, k = (h @ w[p + "q"].T).reshape(n, H, dk), (h @ w[p + "k"].T).reshape(n, G, dk)
+    if cfg.get("unit_norm", True):
+        q, k = rms_unit(q, eps), rms_unit(k, eps)
     v = (h @ w[p + "v"].T).reshape(n, G, dv)
     if cfg.get("v_mix"):
         if first_values is None:
@@ -62,8 +64,11 @@ def attention(h, w, p, cfg, eps, first_values):
     for a in range(H):
         g = a // (H // G)
         s = cap_scores(q[:, a] @ k[:, g].T * cfg["scale"], cfg.get("softcap"))
-        out[:, a] = sink_softmax(s, visible, w[p + "sink"][a]) @ v[:, g]
-    return (out.reshape(n, H * dv) * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T, first_values
+        out[:, a] = sink_softmax(s, visible, w[p + "sink"][a] if cfg.get("has_sink", True) else -np.inf) @ v[:, g]
+    out = out.reshape(n, H * dv)
+    if cfg.get("gate", True):
+        out = out * sigmoid(h @ w[p + "g"].T)
+    return out @ w[p + "o"].T, first_values
 
 
 def feed_forward(h, w, p):
@@ -93,7 +98,7 @@ def random_model(config, seed, bf16=True):
     g = torch.Generator().manual_seed(seed)
 
     def t(*shape, scale=1.0, mean=0.0):
-        a = torch.randn(*shape, generator=g) * scale + mean
+        a = torch.randn(tuple(shape), generator=g) * scale + mean
         return (a.bfloat16() if bf16 else a).float().numpy()
 
     W = config["width"]
