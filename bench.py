@@ -44,6 +44,8 @@ def parse():
     ap.add_argument("--cpu-seconds", type=float, default=12.0)
     ap.add_argument("--no-extras", action="store_true", help="skip extra_configs / plugin_decode / the llama_decode CPU baseline")
     ap.add_argument("--tmp", default=os.environ.get("TMPDIR", "/tmp"), help="where the synthetic GGUF files of the plug-in legs go")
+    ap.add_argument("--design", default="", help="kudirax[:size,size]: prefill / decode throughput and kernel rooflines of the layer-described design at a few sizes, beside a "
+                                                 "llama window of equal size, instead of the headline workload")
     ap.add_argument("--section", default="", help="(internal) run ONE extra leg in this process and print its JSON: prefill_qwen | long_context[:model]")
     return ap.parse_args()
 
@@ -746,6 +748,11 @@ def section_long_context(name="llama3-70b", ctxs=(8192, 32768)):
 
 def main():
     a = parse()
+    if a.design:
+        assert torch.cuda.is_available(), "bench.py needs a HIP device (no CPU fallback)"
+        from prima_cpp_amd import bench_design
+        bench_design.main(a.design, a.steps, a.warmup)
+        return
     if a.section == "prefill_qwen":
         assert torch.cuda.is_available(), "bench.py needs a HIP device (no CPU fallback)"
         section_prefill_qwen()

@@ -40,7 +40,30 @@ template <typename T> __global__ __launch_bounds__(256) void attn_prepare_kernel
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     if ((int) blockIdx.x < n_tok) {
         const int t = blockIdx.x, pos = b.pos[t], page = b.table[(size_t) b.seq[t] * b.table_ld + pos / PM_PAGE], slot = pos % PM_PAGE;
-        for (int i = wave; i < a.H + a.G; i += 4) {
+        const int n = a.H + a.G;
+        int i = wave;
+        if (a.dkp <= 128) for (; i + 12 < n; i += 16) {    // four heads' loads at a time
+            float v[4][2], rs[4];
+            size_t at[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int hd = i + j * 4;
+                at[j] = (size_t) t * a.ldraw + (hd < a.H ? q_off(a, hd) : k_off(a, hd - a.H));
+                v[j][0] = lane < a.dk ? ld_any(a.raw, at[j] + lane, a.raw_type) : 0.0f;
+                v[j][1] = lane + 64 < a.dk ? ld_any(a.raw, at[j] + lane + 64, a.raw_type) : 0.0f;
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                rs[j] = a.flags & PM355_MIX_QK_NORM ? 1.0f / sqrtf(wave_sum(fmaf(v[j][1], v[j][1], v[j][0] * v[j][0])) / (float) a.dk + a.eps) : 1.0f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int hd = i + j * 4;
+                T * dst = hd < a.H ? (T *) a.q + ((size_t) t * a.H + hd) * a.dkp : (T *) a.kc + (((size_t) page * a.G + (hd - a.H)) * PM_PAGE + slot) * a.dkp;
+                dst[lane] = from_f<T>(v[j][0] * rs[j]);
+                if (a.dkp == 128) dst[lane + 64] = from_f<T>(v[j][1] * rs[j]);
+            }
+        }
+        for (; i < n; i += 4) {
             const bool isq = i < a.H;
             const size_t at = (size_t) t * a.ldraw + (isq ? q_off(a, i) : k_off(a, i - a.H));
             const float rs = unit_scale(a, at, a.dk);
@@ -112,11 +135,16 @@ template <typename T> __global__ __launch_bounds__(256) void attn_plain_kernel(p
 
 __device__ __forceinline__ bf16x8 ld_b8(const uint16_t * p) { return __builtin_bit_cast(bf16x8, *(const PM_G u32x4 *) p); }
 
-template <int DK, int DV> __global__ __launch_bounds__(256) void attn_decode_kernel(pm_attn_layer a, pm_batch_dev b, const int32_t * rows, int fused, int splits) {
-    constexpr int KS = DK / 32, VT = DV / 16;
+// values published inside a launch for a workgroup on any XCD: write-through stores, loads that no cache answers
+__device__ __forceinline__ void st_shared(float * p, float v) { __hip_atomic_store((PM_G float *) p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+__device__ __forceinline__ float ld_shared(const float * p) { return __hip_atomic_load((const PM_G float *) p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+
+constexpr int DW = 8;                                      // waves of a decode workgroup: 32 keys each = 256 keys per round
+template <int DK, int DV> __global__ __launch_bounds__(DW * 64) void attn_decode_kernel(pm_attn_layer a, pm_batch_dev b, const int32_t * rows, int fused, int splits) {
+    constexpr int KS = DK / 32, VT = DV / 16, QL = DK / 64;
     extern __shared__ __attribute__((aligned(16))) char smem[];
-    float * acc_l = (float *) smem;                        // [4 waves][16 heads][DV]; its front is the query tile before the key loop
-    float * m_l = acc_l + 4 * 16 * DV, * l_l = m_l + 64;
+    float * acc_l = (float *) smem;                        // [DW waves][16 heads][DV]; its front is the query tile before the key loop
+    float * m_l = acc_l + DW * 16 * DV, * l_l = m_l + DW * 16;
     uint16_t * q_l = (uint16_t *) smem;                    // [16][DK + 8]
     __shared__ int is_last;
     const int R = a.H / a.G, HT = (R + 15) / 16, g = blockIdx.y / HT, h0 = g * R + blockIdx.y % HT * 16, nh = R - blockIdx.y % HT * 16 < 16 ? R - blockIdx.y % HT * 16 : 16;
@@ -126,18 +154,36 @@ template <int DK, int DV> __global__ __launch_bounds__(256) void attn_decode_ker
     // this workgroup's pages
     const int p0 = first / PM_PAGE, np = pos / PM_PAGE - p0 + 1, per = (np + splits - 1) / splits, s = blockIdx.z;
     const int lo = p0 + s * per, hi = p0 + ((s + 1) * per < np ? (s + 1) * per : np);
+    const int krow = 8 * (lr >> 2) + (lr & 3);             // key of score row lr in tile 0 (tile 1: + 4)
+    bf16x8 k0[KS], k1[KS], v[VT];
+    auto load = [&](int c) __attribute__((always_inline)) {          // the keys and values of chunk c (32 keys), matrix-core operands as they lie
+        const size_t at = (size_t) pages[c >> 1] * a.G + g;
+        const uint16_t * kp = (const uint16_t *) a.kc + (at * PM_PAGE + (c & 1) * 32 + krow) * DK + lg * 8;
+        const uint16_t * vp = (const uint16_t *) a.vc + (at * DV + lr) * PM_PAGE + (c & 1) * 32 + lg * 8;
+#pragma unroll
+        for (int i = 0; i < KS; ++i) { k0[i] = ld_b8(kp + i * 32); k1[i] = ld_b8(kp + 4 * DK + i * 32); }
+#pragma unroll
+        for (int i = 0; i < VT; ++i) v[i] = ld_b8(vp + i * 16 * PM_PAGE);
+    };
+    // a wave's first chunk is on its way while the queries are prepared - unless it lies in the page that takes the token's own key and value
+    int c = lo * 2 + wave;
+    const bool any = c < hi * 2, early = any && !(fused && (c >> 1) == pos / PM_PAGE);
+    if (early) load(c);
 
-    for (int h = wave; h < 16; h += 4) {
-        if (h < nh) {
-            const size_t at = (size_t) t * a.ldraw + q_off(a, h0 + h);
-            const float rs = fused ? unit_scale(a, at, a.dk) : 1.0f;
-            for (int d = lane; d < DK; d += 64) {
-                uint16_t v;
-                if (fused) v = d < a.dk ? f2bf(ld_any(a.raw, at + d, a.raw_type) * rs) : (uint16_t) 0;
-                else v = ((const uint16_t *) a.q)[((size_t) t * a.H + h0 + h) * DK + d];
-                q_l[h * (DK + 8) + d] = v;
-            }
-        } else for (int d = lane; d < DK; d += 64) q_l[h * (DK + 8) + d] = 0;
+#pragma unroll
+    for (int i = 0; i < 16 / DW; ++i) {
+        const int h = wave + i * DW;
+        float x[QL], ss = 0.0f;
+        const size_t at = fused ? (size_t) t * a.ldraw + q_off(a, h0 + h) : ((size_t) t * a.H + h0 + h) * DK;
+#pragma unroll
+        for (int j = 0; j < QL; ++j) {
+            const int d = lane + j * 64;
+            x[j] = h >= nh || d >= a.dk ? 0.0f : fused ? ld_any(a.raw, at + d, a.raw_type) : bf2f(((const uint16_t *) a.q)[at + d]);
+            ss = fmaf(x[j], x[j], ss);
+        }
+        const float rs = fused && (a.flags & PM355_MIX_QK_NORM) ? 1.0f / sqrtf(wave_sum(ss) / (float) a.dk + a.eps) : 1.0f;
+#pragma unroll
+        for (int j = 0; j < QL; ++j) q_l[h * (DK + 8) + lane + j * 64] = f2bf(x[j] * rs);
     }
     if (fused && pos / PM_PAGE >= lo && pos / PM_PAGE < hi) {
         // the token's own key and value: the workgroup that attends them stores them first (pages are not shared between splits)
@@ -146,11 +192,12 @@ template <int DK, int DV> __global__ __launch_bounds__(256) void attn_decode_ker
             const size_t kat = (size_t) t * a.ldraw + k_off(a, g);
             const float rs = unit_scale(a, kat, a.dk);
             for (int d = lane; d < a.dk; d += 64) ((uint16_t *) a.kc)[(at * PM_PAGE + pos % PM_PAGE) * DK + d] = f2bf(ld_any(a.raw, kat + d, a.raw_type) * rs);
-        } else for (int d = threadIdx.x - 64; d < a.dv; d += 192)
+        } else for (int d = threadIdx.x - 64; d < a.dv; d += (DW - 1) * 64)
             ((uint16_t *) a.vc)[(at * DV + d) * PM_PAGE + pos % PM_PAGE] = f2bf(mixed_value(a, t, g * a.dv + d, ld_any(a.raw, (size_t) t * a.ldraw + v_off(a, g) + d, a.raw_type)));
-        __threadfence_block();
+        pm_vm_drain();                                     // (stored before any wave of this workgroup passes the barrier and loads them)
     }
     __syncthreads();
+    if (any && !early) load(c);
     bf16x8 q[KS];
 #pragma unroll
     for (int i = 0; i < KS; ++i) q[i] = *(const bf16x8 *) (q_l + lr * (DK + 8) + i * 32 + lg * 8);
@@ -161,18 +208,11 @@ template <int DK, int DV> __global__ __launch_bounds__(256) void attn_decode_ker
     for (int i = 0; i < VT; ++i) acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     float m = NONE, l = 0.0f;
     const float c_in = a.cap > 0.0f ? 2.0f * LOG2E / a.cap : 0.0f;
-    const int krow = 8 * (lr >> 2) + (lr & 3);             // key of score row lr in tile 0 (tile 1: + 4)
-    for (int c = lo * 2 + wave; c < hi * 2; c += 4) {      // 32 keys at a time
+    for (bool loaded = true; c < hi * 2; c += DW) {
         const int key0 = c * 32;
+        if (!loaded) load(c);
+        loaded = false;
         if (key0 > pos || key0 + 31 < first) continue;
-        const size_t at = (size_t) pages[c >> 1] * a.G + g;
-        const uint16_t * kp = (const uint16_t *) a.kc + (at * PM_PAGE + (c & 1) * 32 + krow) * DK + lg * 8;
-        const uint16_t * vp = (const uint16_t *) a.vc + (at * DV + lr) * PM_PAGE + (c & 1) * 32 + lg * 8;
-        bf16x8 k0[KS], k1[KS], v[VT];
-#pragma unroll
-        for (int i = 0; i < KS; ++i) { k0[i] = ld_b8(kp + i * 32); k1[i] = ld_b8(kp + 4 * DK + i * 32); }
-#pragma unroll
-        for (int i = 0; i < VT; ++i) v[i] = ld_b8(vp + i * 16 * PM_PAGE);
         f32x4 s0 = {0.0f, 0.0f, 0.0f, 0.0f}, s1 = s0;
 #pragma unroll
         for (int i = 0; i < KS; ++i) {
@@ -208,60 +248,59 @@ template <int DK, int DV> __global__ __launch_bounds__(256) void attn_decode_ker
     for (int i = 0; i < VT; ++i) *(f32x4 *) (acc_l + (wave * 16 + lr) * DV + i * 16 + lg * 4) = acc[i];
     if (lg == 0) { m_l[wave * 16 + lr] = m; l_l[wave * 16 + lr] = l; }
     __syncthreads();
-    const int sp = splits;
-    float * part = a.part + ((size_t) (blockIdx.x * gridDim.y + blockIdx.y) * sp + s) * 16 * (DV + 2);
-    for (int o = threadIdx.x; o < nh * DV; o += 256) {
+    const bool sink = a.flags & PM355_MIX_SINK;
+    auto store = [&](int h, int d, float o) {
+        if (a.flags & PM355_MIX_OUT_GATE) o *= sigmoid_f(ld_any(a.raw, (size_t) t * a.ldraw + g_off(a, h0 + h) + d, a.raw_type));
+        ((uint16_t *) a.out)[(size_t) t * a.ldo + (h0 + h) * a.dv + d] = f2bf(o);
+    };
+    const size_t slot = (size_t) blockIdx.x * gridDim.y + blockIdx.y;
+    float * part = a.part + slot * splits * 16 * (DV + 2);
+    for (int o = threadIdx.x; o < nh * DV; o += DW * 64) {
         const int h = o / DV, d = o % DV;
-        float M = m_l[h];
+        const float sk = splits == 1 && sink ? a.sink[h0 + h] * LOG2E : NONE;
+        float M = sk;
 #pragma unroll
-        for (int w = 1; w < 4; ++w) M = fmaxf(M, m_l[w * 16 + h]);
-        const bool sink = sp == 1 && (a.flags & PM355_MIX_SINK);
-        const float sk = sink ? a.sink[h0 + h] * LOG2E : NONE;
-        M = fmaxf(M, sk);
-        float v = 0.0f, L = sink ? __builtin_amdgcn_exp2f(sk - M) : 0.0f;
+        for (int w = 0; w < DW; ++w) M = fmaxf(M, m_l[w * 16 + h]);
+        float x = 0.0f, L = splits == 1 && sink ? __builtin_amdgcn_exp2f(sk - M) : 0.0f;
 #pragma unroll
-        for (int w = 0; w < 4; ++w) { const float f = __builtin_amdgcn_exp2f(m_l[w * 16 + h] - M); v += acc_l[(w * 16 + h) * DV + d] * f; L += l_l[w * 16 + h] * f; }
-        if (sp == 1) {
-            if (d < a.dv) {
-                v /= L;
-                if (a.flags & PM355_MIX_OUT_GATE) v *= sigmoid_f(ld_any(a.raw, (size_t) t * a.ldraw + g_off(a, h0 + h) + d, a.raw_type));
-                ((uint16_t *) a.out)[(size_t) t * a.ldo + (h0 + h) * a.dv + d] = f2bf(v);
-            }
-        } else {
-            part[h * (DV + 2) + d] = v;
-            if (d == 0) { part[h * (DV + 2) + DV] = M; part[h * (DV + 2) + DV + 1] = L; }
+        for (int w = 0; w < DW; ++w) { const float f = __builtin_amdgcn_exp2f(m_l[w * 16 + h] - M); x += acc_l[(w * 16 + h) * DV + d] * f; L += l_l[w * 16 + h] * f; }
+        if (splits == 1) { if (d < a.dv) store(h, d, x / L); }
+        else {
+            float * r = part + (s * 16 + h) * (DV + 2);
+            st_shared(r + d, x);
+            if (d == 0) { st_shared(r + DV, M); st_shared(r + DV + 1, L); }
         }
     }
-    if (sp == 1) return;
-    // partials out, ticket; the last split of this (token, KV head) merges all of them and re-arms the ticket
-    __threadfence();
+    if (splits == 1) return;
+    // partials out, then a ticket; the last split of this (token, KV head) merges all of them and re-arms the ticket
+    pm_vm_drain();
     __syncthreads();
     if (threadIdx.x == 0) {
-        unsigned * tk = a.ticket + blockIdx.x * gridDim.y + blockIdx.y;
-        const unsigned n = __hip_atomic_fetch_add(tk, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
-        is_last = n == (unsigned) sp - 1;
+        unsigned * tk = a.ticket + slot;
+        is_last = __hip_atomic_fetch_add(tk, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (unsigned) splits - 1;
         if (is_last) __hip_atomic_store(tk, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     }
     __syncthreads();
     if (!is_last) return;
-    __threadfence();
-    const float * all = a.part + (size_t) (blockIdx.x * gridDim.y + blockIdx.y) * sp * 16 * (DV + 2);
-    for (int o = threadIdx.x; o < nh * DV; o += 256) {
+    float * ml = acc_l;                                    // [splits][16][2]
+    for (int o = threadIdx.x; o < splits * 32; o += DW * 64) if ((o >> 1 & 15) < nh) ml[o] = ld_shared(part + (o >> 1) * (DV + 2) + DV + (o & 1));
+    __syncthreads();
+    for (int o = threadIdx.x; o < nh * DV; o += DW * 64) {
         const int h = o / DV, d = o % DV;
         if (d >= a.dv) continue;
-        const bool sink = a.flags & PM355_MIX_SINK;
         const float sk = sink ? a.sink[h0 + h] * LOG2E : NONE;
         float M = sk;
-        for (int i = 0; i < sp; ++i) M = fmaxf(M, all[(i * 16 + h) * (DV + 2) + DV]);
-        float v = 0.0f, L = sink ? __builtin_amdgcn_exp2f(sk - M) : 0.0f;
-        for (int i = 0; i < sp; ++i) {
-            const float * r = all + (i * 16 + h) * (DV + 2);
-            const float f = __builtin_amdgcn_exp2f(r[DV] - M);
-            v += r[d] * f; L += r[DV + 1] * f;
+        for (int i = 0; i < splits; ++i) M = fmaxf(M, ml[(i * 16 + h) * 2]);
+        float x = 0.0f, L = sink ? __builtin_amdgcn_exp2f(sk - M) : 0.0f;
+        for (int i0 = 0; i0 < splits; i0 += 8) {
+            float r[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) r[i] = ld_shared(part + ((i0 + i < splits ? i0 + i : splits - 1) * 16 + h) * (DV + 2) + d);
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+                if (i0 + i < splits) { const float f = __builtin_amdgcn_exp2f(ml[((i0 + i) * 16 + h) * 2] - M); x += r[i] * f; L += ml[((i0 + i) * 16 + h) * 2 + 1] * f; }
         }
-        v /= L;
-        if (a.flags & PM355_MIX_OUT_GATE) v *= sigmoid_f(ld_any(a.raw, (size_t) t * a.ldraw + g_off(a, h0 + h) + d, a.raw_type));
-        ((uint16_t *) a.out)[(size_t) t * a.ldo + (h0 + h) * a.dv + d] = f2bf(v);
+        store(h, d, x / L);
     }
 }
 
@@ -438,9 +477,10 @@ template <int DK, int DV> int launch_tiles(const pm_attn_layer & a, const pm_bat
 }
 template <int DK, int DV> int launch_decode(const pm_attn_layer & a, const pm_batch_dev & b, const int32_t * rows, int n, int fused, int splits, hipStream_t st) {
     const int R = a.H / a.G, HT = (R + 15) / 16;
-    const size_t lds = (size_t) 4 * 16 * DV * 4 + 512 > (size_t) 16 * (DK + 8) * 2 ? (size_t) 4 * 16 * DV * 4 + 512 : (size_t) 16 * (DK + 8) * 2;
+    constexpr size_t lds = (size_t) DW * 16 * (DV + 2) * 4;      // (covers the query tile: 16 x (DK + 8) halves, and the merge's 64 x 32 floats)
+    static_assert(lds >= (size_t) 16 * (DK + 8) * 2 && lds >= 64 * 32 * 4, "LDS");
     pm_allow_big_lds((const void *) attn_decode_kernel<DK, DV>, lds);
-    hipLaunchKernelGGL((attn_decode_kernel<DK, DV>), dim3(n, a.G * HT, splits), dim3(256), lds, st, a, b, rows, fused, splits);
+    hipLaunchKernelGGL((attn_decode_kernel<DK, DV>), dim3(n, a.G * HT, splits), dim3(DW * 64), lds, st, a, b, rows, fused, splits);
     return 0;
 }
 

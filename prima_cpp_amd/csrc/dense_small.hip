@@ -6,6 +6,7 @@
 #include "pm355_dense.h"
 #include "pm355_kernels.h"
 #include "../../include/prima_mi355.h"
+#include <type_traits>
 
 namespace {
 
@@ -74,8 +75,9 @@ template <typename T, int TP> __device__ __forceinline__ void add_norm_prologue(
     __syncthreads();
 }
 
-template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) void dense_small_kernel(SmallP p) {
-    constexpr int PB = Frag<T>::PER_BLOCK, U = (sizeof(T) == 2 ? 4 : 2), EPL = 16 / sizeof(T);      // U blocks per load group, elements per 16 bytes
+template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void dense_small_kernel(SmallP p) {
+    // U blocks per load group (eight 16-byte loads per lane; two groups are in flight), EPL elements per 16 bytes
+    constexpr int PB = Frag<T>::PER_BLOCK, EPL = 16 / sizeof(T), UG = 8 / (PB * RM) / (NT == 4 ? 2 : 1), U = UG < 1 ? 1 : UG;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     float * red = (float *) smem;                                                                  // [8 waves][NT][RM][16 tokens][16 rows]
     const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
@@ -84,19 +86,18 @@ template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) 
     const T * wrow[RM];
 #pragma unroll
     for (int m = 0; m < RM; ++m) wrow[m] = (const T *) p.W + (size_t) (r0 + m * 16 + lr) * p.K + g * EPL;
-    auto load_a = [&](u32x4 (&a)[RM][PB], int i) __attribute__((always_inline)) {
-        const int k = (wave + i * 8) << 6;
+    auto load = [&](u32x4 (&a)[U][RM][PB], int grp) __attribute__((always_inline)) {
 #pragma unroll
-        for (int m = 0; m < RM; ++m)
+        for (int u = 0; u < U; ++u) {
+            const int i = grp * U + u, k = (wave + (i < mine ? i : mine - 1) * 8) << 6;            // (past the end: the last block again, not multiplied)
 #pragma unroll
-            for (int s = 0; s < PB; ++s) a[m][s] = ld_nt16(wrow[m] + k + s * (64 / PB));
+            for (int m = 0; m < RM; ++m)
+#pragma unroll
+                for (int s = 0; s < PB; ++s) a[u][m][s] = ld_nt16(wrow[m] + k + s * (64 / PB));
+        }
     };
-    u32x4 a[U][RM][PB];
-    const bool first = mine >= U;                          // the first group's weights are on their way while the prologue runs
-    if (TP && first) {
-#pragma unroll
-        for (int u = 0; u < U; ++u) load_a(a[u], u);
-    }
+    u32x4 wa[U][RM][PB], wb[U][RM][PB];
+    if (mine > 0) load(wa, 0);                             // the first weights are on their way while the prologue runs
     const T * arow[NT];
     if (TP) {
         const int ldl = p.K + EPL;
@@ -112,27 +113,27 @@ template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) 
     for (int n = 0; n < NT; ++n)
 #pragma unroll
         for (int m = 0; m < RM; ++m) acc[n][m] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-    auto mma_block = [&](const u32x4 (&w)[RM][PB], int i) __attribute__((always_inline)) {
-        const int k = (wave + i * 8) << 6;
+    auto mma = [&](const u32x4 (&w)[U][RM][PB], int grp, bool full) __attribute__((always_inline)) {
 #pragma unroll
-        for (int s = 0; s < PB; ++s)
+        for (int u = 0; u < U; ++u) {
+            const int i = grp * U + u, k = (wave + i * 8) << 6;
+            if (!full && i >= mine) break;
 #pragma unroll
-            for (int n = 0; n < NT; ++n) {
-                const u32x4 b = TP ? *(const u32x4 *) (arow[n] + k + s * (64 / PB)) : *(const PM_G u32x4 *) (arow[n] + k + s * (64 / PB));
+            for (int s = 0; s < PB; ++s)
 #pragma unroll
-                for (int m = 0; m < RM; ++m) acc[n][m] = Frag<T>::mma(w[m][s], b, acc[n][m]);
-            }
-    };
-    int i = 0;
-    for (; i + U <= mine; i += U) {
-        if (!(TP && i == 0)) {
+                for (int n = 0; n < NT; ++n) {
+                    const u32x4 b = TP ? *(const u32x4 *) (arow[n] + k + s * (64 / PB)) : *(const PM_G u32x4 *) (arow[n] + k + s * (64 / PB));
 #pragma unroll
-            for (int u = 0; u < U; ++u) load_a(a[u], i + u);
+                    for (int m = 0; m < RM; ++m) acc[n][m] = Frag<T>::mma(w[u][m][s], b, acc[n][m]);
+                }
         }
-#pragma unroll
-        for (int u = 0; u < U; ++u) mma_block(a[u], i + u);
-    }
-    for (; i < mine; ++i) { load_a(a[0], i); mma_block(a[0], i); }
+    };
+    // two register sets, the next group's loads in front of this group's products
+    const int ng = (mine + U - 1) / U;
+    int g2 = 0;
+    for (; g2 + 2 < ng; g2 += 2) { load(wb, g2 + 1); mma(wa, g2, true); load(wa, g2 + 2); mma(wb, g2 + 1, true); }
+    if (ng - g2 == 2) { load(wb, g2 + 1); mma(wa, g2, true); mma(wb, g2 + 1, false); }
+    else if (ng - g2 == 1) mma(wa, g2, false);
 #pragma unroll
     for (int n = 0; n < NT; ++n)
 #pragma unroll
@@ -162,13 +163,19 @@ template <typename T, int NT, int RM, int TP> int launch(const SmallP & p, int N
 template <typename T> int launch_type(const pm_dense_args & a, const SmallP & p, hipStream_t st) {
     const int N = (a.n_store + 63) / 64 * 64;
     if (a.pro) {
+        // every workgroup runs the prologue: few enough of them that all are resident (two per CU)
         if (!pm_dense_pro_ok(a.T, a.pro->width)) return PM355_E_UNSUPPORTED;
-        return a.T == 1 ? launch<T, 1, 1, 1>(p, N, st) : a.T == 2 ? launch<T, 1, 1, 2>(p, N, st) : launch<T, 1, 1, 4>(p, N, st);
+        auto go = [&](auto rm) {
+            constexpr int RM = decltype(rm)::value;
+            return a.T == 1 ? launch<T, 1, RM, 1>(p, N, st) : a.T == 2 ? launch<T, 1, RM, 2>(p, N, st) : launch<T, 1, RM, 4>(p, N, st);
+        };
+        return N / 16 <= 512 ? go(std::integral_constant<int, 1>()) : N / 32 <= 512 ? go(std::integral_constant<int, 2>()) : go(std::integral_constant<int, 4>());
     }
     const bool wide = N / 32 >= 512;
     if (a.T <= 16) return wide ? launch<T, 1, 2, 0>(p, N, st) : launch<T, 1, 1, 0>(p, N, st);
     if (a.T <= 32) return wide ? launch<T, 2, 2, 0>(p, N, st) : launch<T, 2, 1, 0>(p, N, st);
-    return wide ? launch<T, 4, 2, 0>(p, N, st) : launch<T, 4, 1, 0>(p, N, st);
+    if constexpr (sizeof(T) == 2) if (wide) return launch<T, 4, 2, 0>(p, N, st);
+    return launch<T, 4, 1, 0>(p, N, st);
 }
 
 } // namespace

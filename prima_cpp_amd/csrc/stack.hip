@@ -94,6 +94,12 @@ struct pm_stack : pm355_model {
     int locate(int kind, int layer, void ** dst, int64_t & rows, int & K, int & Kp, int & type, float ** scalar);
     int set_tensor(int kind, int layer, int type, const void * host, size_t nbytes) override;
     int fill_tensor(int kind, int layer, int type, uint64_t seed, float scale) override;
+    void * tensor_ptr(int kind, int layer, int * type_out) override {
+        void * dst = nullptr; int64_t rows; int K, Kp, dt; float * scalar;
+        if (locate(kind, layer, &dst, rows, K, Kp, dt, &scalar) || scalar) return nullptr;
+        if (type_out) *type_out = dt;
+        return dst;
+    }
     int finalize(int max_tokens_, int n_seq) override { return finalize_pool(max_tokens_, n_seq, (int64_t) n_seq * 4096); }
     int finalize_pool(int max_tokens_, int n_seq, int64_t pool_tokens) override;
     size_t weight_bytes() const override { return n_weight_bytes - (size_t) embed.Kp * embed.Np * pm_dense_bytes(d.type); }
