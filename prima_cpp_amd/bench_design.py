@@ -114,7 +114,7 @@ def kernels_design(m, z):
         y = torch.empty(1, N, dtype=torch.bfloat16 if k == "up" else torch.float32, device="cuda")
         bias = torch.zeros(N, device="cuda") if k in ("up", "down") else None
         x = torch.randn(1, K, device="cuda").bfloat16()
-        pro = k in ("proj", "up") and W <= 8192
+        pro = k in ("proj", "up") and W <= 2048           # (wider rows: a norm launch of its own, as the engine does it)
         if pro:
             us = timed(lambda: [ops.dense_mul_mat_norm(a, r, dl, nw, nb, 1e-5, r2, y, W, bias=bias, act=int(k == "up")) for a in w[k]], n)
         else:
@@ -157,6 +157,8 @@ def kernels_design(m, z):
     out["prefill"]["attention_small_cap"] = row(timed(lambda: [attn(i, 18, PROMPT, 15.0) for i in range(4)], 4), flop, MFMA)
     byt = PROMPT * (Np - H * d + H * d + 2 * G * d) * 2
     out["prefill"]["unit_norm_and_store"] = row(timed(lambda: [attn(i, 0, PROMPT) for i in range(4)], 4), byt, HBM)
+    r1, x1 = torch.randn(1, W, device="cuda"), torch.empty(1, W, dtype=torch.bfloat16, device="cuda")
+    out["decode"]["add_norm"] = row(timed(lambda: [ops.add_layer_norm(r1, dl, nw, nb, 1e-5, W, x1) for _ in range(8)], 8), W * 22, HBM)
     rr, dd, xb = torch.randn(PROMPT, W, device="cuda"), torch.randn(PROMPT, W, device="cuda"), torch.empty(PROMPT, W, dtype=torch.bfloat16, device="cuda")
     out["prefill"]["add_norm"] = row(timed(lambda: [ops.add_layer_norm(rr, dd, nw, nb, 1e-5, W, xb) for _ in range(4)], 4), PROMPT * W * 14, HBM)
     return out
@@ -229,10 +231,18 @@ def kernels_window(w, z):
     out["decode"]["attention"] = dict(row(us, 2 * CTX * G * d * 2, HBM), keys=CTX)
     us = timed(lambda: [check(pre(ptr(q), ptr(kc[i]), ptr(vc[i]), ptr(pos[1:]), ptr(o), PROMPT, H, G, d, CTX, 0.1, st()), "attention") for i in range(4)], 4)
     out["prefill"]["attention"] = row(us, 4.0 * d * H * PROMPT * (PROMPT + 1) / 2, MFMA)
+    rp = ops.RopeParams(n_dims=d, mode=0, n_ctx_orig=8192, freq_base=500000.0, freq_scale=1.0, ext_factor=0.0, attn_factor=1.0, beta_fast=32.0, beta_slow=1.0)
+    rope = L.declare("pm355_rope_kv_store", C.c_int, [C.c_void_p] * 9 + [C.c_int] * 5 + [C.c_void_p, C.c_void_p])
+    k, v = torch.randn(PROMPT, G * d, device="cuda"), torch.randn(PROMPT, G * d, device="cuda")
+    us = timed(lambda: [check(rope(ptr(q), ptr(k), ptr(v), ptr(o), None, ptr(kc[i]), ptr(vc[i]), ptr(pos[1:]), None, PROMPT, H, G, d, CTX, C.addressof(rp), st()), "rope") for i in range(4)], 4)
+    out["prefill"]["rope_and_store"] = row(us, PROMPT * (H * d * 8 + G * d * 12), HBM)
+    norm = L.declare("pm355_rms_norm", C.c_int, [C.c_void_p] * 4 + [C.c_int64, C.c_int64, C.c_float, C.c_void_p])
+    r, rn, nw = torch.randn(PROMPT, W, device="cuda"), torch.empty(PROMPT, W, device="cuda"), torch.ones(W, device="cuda")
+    out["prefill"]["norm"] = row(timed(lambda: [check(norm(ptr(r), ptr(nw), ptr(rn), None, W, PROMPT, 1e-5, st()), "norm") for _ in range(4)], 4), PROMPT * W * 8, HBM)
     return out
 
 
-LIKE = {"proj": "qkv", "out": "out", "up": "gate|up", "down": "down", "attention": "attention", "attention_small_cap": "attention"}
+LIKE = {"proj": "qkv", "out": "out", "up": "gate|up", "down": "down", "attention": "attention", "attention_small_cap": "attention", "unit_norm_and_store": "rope_and_store", "add_norm": "norm"}
 
 
 def main(what, steps, warmup):
@@ -250,7 +260,7 @@ def main(what, steps, warmup):
         b = {"weights": "Q8_0", "throughput": throughput_window(w, z, steps, warmup), "kernels": kernels_window(w, z), "weight_bytes": w.weight_bytes}
         w.close()
         torch.cuda.empty_cache()
-        far = {ph: {k: round(b["kernels"][ph][LIKE[k]]["of_roofline"] / v["of_roofline"], 2) for k, v in a["kernels"][ph].items() if k in LIKE} for ph in ("decode", "prefill")}
+        far = {ph: {k: round(b["kernels"][ph][LIKE[k]]["of_roofline"] / v["of_roofline"], 2) for k, v in a["kernels"][ph].items() if LIKE.get(k) in b["kernels"][ph]} for ph in ("decode", "prefill")}
         res[size] = {"kudirax": a, "llama_same_size": b, "times_further_from_roofline_than_llama": far}
         print("design %s: %s" % (size, json.dumps(far)), flush=True)
     print(json.dumps({"metric": "kudirax_decode_tokens_per_s", "value": next(iter(res.values()))["kudirax"]["throughput"]["decode_1"]["tok/s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,

@@ -42,24 +42,42 @@ __device__ __forceinline__ float block_sum(float v, float * red) {
     return s;
 }
 
-// one row per workgroup. RES: x[row] += layer_norm(y[row]) and out = the sum in T; else out[row] = layer_norm(x[rows[row]]) in T
-template <bool RES> __global__ __launch_bounds__(256) void layer_norm_kernel(int type, float * x, const float * y, int ldx, int ldy, const int32_t * rows, const float * w,
-                                                                            const float * b, float eps, int width, void * out, int ldo) {
+// one row per workgroup. RES: x[row] += layer_norm(y[row]) and out = the sum in T; else out[row] = layer_norm(x[rows[row]]) in T. VP > 0: the row and everything that joins
+// it are requested at once, VP values per lane; 0: any width, row in LDS
+template <bool RES, int NTH, int VP> __global__ __launch_bounds__(NTH) void layer_norm_kernel(int type, float * x, const float * y, int ldx, int ldy, const int32_t * rows, const float * w,
+                                                                                             const float * b, float eps, int width, void * out, int ldo) {
     extern __shared__ __attribute__((aligned(16))) float row[];
-    __shared__ float red[4];
+    __shared__ float red[NTH / 64];
+    constexpr int N = VP ? VP : 1;
     const int r = blockIdx.x;
     const float * src = RES ? y + (size_t) r * ldy : x + (size_t) (rows ? rows[r] : r) * ldx;
-    float s = 0.0f;
-    for (int c = threadIdx.x; c < width; c += 256) { const float v = src[c]; row[c] = v; s += v; }
+    float v[N], xv[N], wv[N], bv[N], s = 0.0f;
+    if (VP) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const int c = i * NTH + threadIdx.x, cc = c < width ? c : width - 1;
+            v[i] = ld_g(src + cc); wv[i] = ld_g(w + cc); bv[i] = ld_g(b + cc);
+            xv[i] = RES ? ld_g(x + (size_t) r * ldx + cc) : 0.0f;
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) s += i * NTH + (int) threadIdx.x < width ? v[i] : 0.0f;
+    } else for (int c = threadIdx.x; c < width; c += NTH) { const float f = src[c]; row[c] = f; s += f; }
     const float mean = block_sum(s, red) / (float) width;
     float s2 = 0.0f;
-    for (int c = threadIdx.x; c < width; c += 256) { const float d = row[c] - mean; s2 = fmaf(d, d, s2); }
+    if (VP) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) { const float d = i * NTH + (int) threadIdx.x < width ? v[i] - mean : 0.0f; s2 = fmaf(d, d, s2); }
+    } else for (int c = threadIdx.x; c < width; c += NTH) { const float d = row[c] - mean; s2 = fmaf(d, d, s2); }
     const float rs = 1.0f / sqrtf(block_sum(s2, red) / (float) width + eps);
-    for (int c = threadIdx.x; c < width; c += 256) {
-        float v = (row[c] - mean) * rs * w[c] + b[c];
-        if (RES) { v = x[(size_t) r * ldx + c] + v; x[(size_t) r * ldx + c] = v; }
-        if (out) st_type(out, (size_t) r * ldo + c, type, v);
-    }
+    auto put = [&](int c, float f, float xo, float wo, float bo) __attribute__((always_inline)) {
+        float o = (f - mean) * rs * wo + bo;
+        if (RES) { o = xo + o; x[(size_t) r * ldx + c] = o; }
+        if (out) st_type(out, (size_t) r * ldo + c, type, o);
+    };
+    if (VP) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) { const int c = i * NTH + threadIdx.x; if (c < width) put(c, v[i], xv[i], wv[i], bv[i]); }
+    } else for (int c = threadIdx.x; c < width; c += NTH) put(c, row[c], RES ? x[(size_t) r * ldx + c] : 0.0f, w[c], b[c]);
 }
 
 // index of the first maximum of every row (src/llama-sampling.cpp:390-397), also kept per sequence for the next step
@@ -95,14 +113,24 @@ void pm_launch_dense_fill(int type, void * dst, int K, int64_t N, int Kp, uint64
 void pm_launch_stack_embed(int type, const void * embed, int Kp, int width, const pm_batch_dev & b, int T, float * x, void * xb, hipStream_t st) {
     hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, st, type, embed, Kp, width, b, x, xb);
 }
+template <bool RES> static void launch_norm(int type, float * x, const float * y, int ldx, int ldy, const int32_t * rows, const float * w, const float * b, float eps, int width, int n_rows,
+                                            void * out, int ldo, hipStream_t st) {
+    auto go = [&](auto kern, int threads, size_t lds) {
+        pm_allow_big_lds((const void *) kern, lds);
+        hipLaunchKernelGGL(kern, dim3(n_rows), dim3(threads), lds, st, type, x, y, ldx, ldy, rows, w, b, eps, width, out, ldo);
+    };
+    if (width <= 1024) go(layer_norm_kernel<RES, 256, 4>, 256, 0);
+    else if (width <= 4096 && n_rows > 512) go(layer_norm_kernel<RES, 256, 16>, 256, 0);
+    else if (width <= 4096) go(layer_norm_kernel<RES, 1024, 4>, 1024, 0);
+    else if (width <= 8192) go(layer_norm_kernel<RES, 1024, 8>, 1024, 0);
+    else go(layer_norm_kernel<RES, 1024, 0>, 1024, (size_t) width * 4);
+}
 void pm_launch_add_layer_norm(int type, float * x, const float * y, int ldx, int ldy, const float * w, const float * b, float eps, int width, int n_rows, void * xb, hipStream_t st) {
-    pm_allow_big_lds((const void *) layer_norm_kernel<true>, (size_t) width * 4);
-    hipLaunchKernelGGL(layer_norm_kernel<true>, dim3(n_rows), dim3(256), (size_t) width * 4, st, type, x, y, ldx, ldy, nullptr, w, b, eps, width, xb, ldx);
+    launch_norm<true>(type, x, y, ldx, ldy, nullptr, w, b, eps, width, n_rows, xb, ldx, st);
 }
 void pm_launch_layer_norm_rows(int type, const float * x, int ldx, const int32_t * rows, const float * w, const float * b, float eps, int width, int n_rows, void * out, int ldo,
                                hipStream_t st) {
-    pm_allow_big_lds((const void *) layer_norm_kernel<false>, (size_t) width * 4);
-    hipLaunchKernelGGL(layer_norm_kernel<false>, dim3(n_rows), dim3(256), (size_t) width * 4, st, type, (float *) x, nullptr, ldx, 0, rows, w, b, eps, width, out, ldo);
+    launch_norm<false>(type, (float *) x, nullptr, ldx, 0, rows, w, b, eps, width, n_rows, out, ldo, st);
 }
 void pm_launch_argmax_rows(const float * logits, int n, int n_rows, int32_t * out, const int32_t * seq_of_row, int32_t * last, hipStream_t st) {
     hipLaunchKernelGGL(argmax_rows_kernel, dim3(n_rows), dim3(1024), 0, st, logits, n, out, seq_of_row, last);

@@ -6,7 +6,6 @@
 #include "pm355_dense.h"
 #include "pm355_kernels.h"
 #include "../../include/prima_mi355.h"
-#include <type_traits>
 
 namespace {
 
@@ -14,7 +13,9 @@ struct SmallP {
     const void * W; const void * act; void * y; const float * bias; pm_add_norm pro;
     int K, T, lda, ldy, y_type, n_store, act_fn;
 };
-constexpr int PRO_MAX = 8192;                              // width x tokens (rounded up to a power of two) that the prologue holds in registers
+// The norm prologue pays where a launch is short: up to this width x tokens (rounded up to a power of two). Wider rows cost every workgroup more than one norm launch does
+// (width 2048: 8.3 us against 6.7 + 3.0; 4096: 20.8 against 15.5 + 4.2; 8192: 87 against 57 + 7)
+constexpr int PRO_MAX = 2048;
 
 template <typename T> struct Frag;                         // one 16-byte load per lane
 template <> struct Frag<uint16_t> {
@@ -33,87 +34,124 @@ template <> struct Frag<float> {
     }
 };
 
-// rows r of [0, T): x + layer_norm(y) -> LDS (T, stride ldl) and, from workgroup 0, the residual stream. 8 / TP waves per token.
-template <typename T, int TP> __device__ __forceinline__ void add_norm_prologue(const SmallP & p, T * rows, int ldl, float * red) {
-    constexpr int NW = 8 / TP, VPL = PRO_MAX / TP / (NW * 64);
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = wave / NW, l = (wave % NW) * 64 + lane;
-    const pm_add_norm & q = p.pro;
-    const bool on = t < p.T;
-    const int tt = on ? t : 0;
-    float v[VPL];
-    float s = 0.0f;
+// x + layer_norm(y) of token wave / (8 / TP) in VP values per lane: everything the rows need is requested before the first weights (loads return in order), the sums run
+// while those are on their way. Result -> LDS (T, stride ldl) and, from workgroup 0, the residual stream.
+template <typename T, int TP> struct AddNorm {
+    static constexpr int NW = 8 / TP, VP = PRO_MAX / 512;
+    float y[VP], x[VP], w[VP], b[VP];
+    int t, l;
+    __device__ __forceinline__ void request(const SmallP & p, int wave, int lane) {
+        const pm_add_norm & q = p.pro;
+        t = wave / NW; l = (wave % NW) * 64 + lane;
+        const int tt = t < p.T ? t : 0;
 #pragma unroll
-    for (int i = 0; i < VPL; ++i) { const int c = i * NW * 64 + l; v[i] = c < q.width ? q.y[(size_t) tt * q.ldy + c] : 0.0f; s += v[i]; }
-    s = wave_sum(s);
-    if (lane == 0) red[wave] = s;
-    __syncthreads();
-    float mean = 0.0f;
-#pragma unroll
-    for (int i = 0; i < NW; ++i) mean += red[t * NW + i];
-    mean /= (float) q.width;
-    float s2 = 0.0f;
-#pragma unroll
-    for (int i = 0; i < VPL; ++i) { const int c = i * NW * 64 + l; const float d = c < q.width ? v[i] - mean : 0.0f; s2 = fmaf(d, d, s2); }
-    s2 = wave_sum(s2);
-    if (lane == 0) red[8 + wave] = s2;
-    __syncthreads();
-    float var = 0.0f;
-#pragma unroll
-    for (int i = 0; i < NW; ++i) var += red[8 + t * NW + i];
-    const float rs = 1.0f / sqrtf(var / (float) q.width + q.eps);
-    if (on) {
-#pragma unroll
-        for (int i = 0; i < VPL; ++i) {
-            const int c = i * NW * 64 + l;
-            if (c < q.width) {
-                const float x = q.x[(size_t) t * q.ldx + c] + ((v[i] - mean) * rs * q.w[c] + q.b[c]);
-                rows[t * ldl + c] = from_f<T>(x);
-                if (blockIdx.x == 0) q.x_out[(size_t) t * q.ldo + c] = x;
-            } else if (c < p.K) rows[t * ldl + c] = from_f<T>(0.0f);
+        for (int i = 0; i < VP; ++i) {
+            const int c = i * NW * 64 + l, cc = c < q.width ? c : q.width - 1;
+            y[i] = ld_g(q.y + (size_t) tt * q.ldy + cc);
+            x[i] = ld_g(q.x + (size_t) tt * q.ldx + cc);
+            w[i] = ld_g(q.w + cc);
+            b[i] = ld_g(q.b + cc);
         }
     }
-    __syncthreads();
-}
+    __device__ __forceinline__ void finish(const SmallP & p, T * rows, int ldl, float * red, int wave, int lane) {
+        const pm_add_norm & q = p.pro;
+        float s = 0.0f;
+#pragma unroll
+        for (int i = 0; i < VP; ++i) s += i * NW * 64 + l < q.width ? y[i] : 0.0f;
+        s = wave_sum(s);
+        if (lane == 0) red[wave] = s;
+        __syncthreads();
+        float mean = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) mean += red[t * NW + i];
+        mean /= (float) q.width;
+        float s2 = 0.0f;
+#pragma unroll
+        for (int i = 0; i < VP; ++i) { const float d = i * NW * 64 + l < q.width ? y[i] - mean : 0.0f; s2 = fmaf(d, d, s2); }
+        s2 = wave_sum(s2);
+        if (lane == 0) red[8 + wave] = s2;
+        __syncthreads();
+        float var = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) var += red[8 + t * NW + i];
+        const float rs = 1.0f / sqrtf(var / (float) q.width + q.eps);
+        if (t < p.T) {
+#pragma unroll
+            for (int i = 0; i < VP; ++i) {
+                const int c = i * NW * 64 + l;
+                if (c < q.width) {
+                    const float v = x[i] + ((y[i] - mean) * rs * w[i] + b[i]);
+                    rows[t * ldl + c] = from_f<T>(v);
+                    if (blockIdx.x == 0) q.x_out[(size_t) t * q.ldo + c] = v;
+                } else if (c < p.K) rows[t * ldl + c] = from_f<T>(0.0f);
+            }
+        }
+        __syncthreads();
+    }
+};
 
-template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void dense_small_kernel(SmallP p) {
-    // U blocks per load group (eight 16-byte loads per lane; two groups are in flight), EPL elements per 16 bytes
-    constexpr int PB = Frag<T>::PER_BLOCK, EPL = 16 / sizeof(T), UG = 8 / (PB * RM) / (NT == 4 ? 2 : 1), U = UG < 1 ? 1 : UG;
+// SRC, where the activations come from: 0 global memory (they ride in the load groups: the vector-memory counter is in order, a later load must not be waited for in front
+// of an earlier one), -1 LDS (copied once), 1 / 2 / 4 the norm prologue for that many tokens (LDS).
+// LINE (bf16, activations in LDS, up to 8 tokens): the 16 tile rows are 8 rows of W x 2 halves of a 64-k block and the 16 columns 8 tokens x the same 2 halves, so that one
+// load instruction covers whole 128-byte lines (a line that two instructions touch is requested twice); of the result the blocks with equal halves count.
+template <typename T, int NT, int RM, int SRC> __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void dense_small_kernel(SmallP p) {
+    constexpr bool LINE = sizeof(T) == 2 && SRC != 0;
+    constexpr int ROWS = LINE ? 8 : 16, TOK = LINE ? 8 : 16, EPL = 16 / sizeof(T);
+    // PB loads per lane and 64-k block, U blocks per load group: about eight 16-byte weight loads per lane, two groups in flight
+    constexpr int PB = LINE ? 1 : Frag<T>::PER_BLOCK, NB = SRC == 0 ? NT : 0, UG = 8 / (PB * (RM + NB)), U = UG < 1 ? 1 : UG;
+    constexpr bool TWO = NB < 4;                           // (NT = 4: one group, its registers are taken by the products)
     extern __shared__ __attribute__((aligned(16))) char smem[];
-    float * red = (float *) smem;                                                                  // [8 waves][NT][RM][16 tokens][16 rows]
+    float * red = (float *) smem;                                                                  // [8 waves][NT][RM][16 columns][16 rows]
     const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
-    const int r0 = blockIdx.x * 16 * RM, t0 = blockIdx.y * 16 * NT;
+    const int r0 = blockIdx.x * ROWS * RM, t0 = blockIdx.y * TOK * NT;
     const int nblk = p.K >> 6, mine = (nblk - wave + 7) >> 3;                                      // 64-k blocks wave, wave + 8, ..
+    const int koff = (LINE ? (lr >> 3) * 32 : 0) + g * EPL;
     const T * wrow[RM];
 #pragma unroll
-    for (int m = 0; m < RM; ++m) wrow[m] = (const T *) p.W + (size_t) (r0 + m * 16 + lr) * p.K + g * EPL;
-    auto load = [&](u32x4 (&a)[U][RM][PB], int grp) __attribute__((always_inline)) {
+    for (int m = 0; m < RM; ++m) wrow[m] = (const T *) p.W + (size_t) (r0 + m * ROWS + lr % ROWS) * p.K + koff;
+    const T * arow[NT];
+    if (SRC == 0) {
+#pragma unroll
+        for (int n = 0; n < NT; ++n) { const int t = t0 + n * 16 + lr; arow[n] = (const T *) p.act + (size_t) (t < p.T ? t : p.T - 1) * p.lda + koff; }
+    }
+    struct Group { u32x4 w[U][RM][PB], x[U][NB ? NB : 1][PB]; };
+    auto load = [&](Group & a, int grp) __attribute__((always_inline)) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const int i = grp * U + u, k = (wave + (i < mine ? i : mine - 1) * 8) << 6;            // (past the end: the last block again, not multiplied)
 #pragma unroll
-            for (int m = 0; m < RM; ++m)
+            for (int s = 0; s < PB; ++s) {
 #pragma unroll
-                for (int s = 0; s < PB; ++s) a[u][m][s] = ld_nt16(wrow[m] + k + s * (64 / PB));
+                for (int n = 0; n < NB; ++n) a.x[u][n][s] = *(const PM_G u32x4 *) (arow[n] + k + s * (64 / PB));
+#pragma unroll
+                for (int m = 0; m < RM; ++m) a.w[u][m][s] = ld_nt16(wrow[m] + k + s * (64 / PB));
+            }
         }
     };
-    u32x4 wa[U][RM][PB], wb[U][RM][PB];
-    if (mine > 0) load(wa, 0);                             // the first weights are on their way while the prologue runs
-    const T * arow[NT];
-    if (TP) {
+    AddNorm<T, SRC < 1 ? 1 : SRC> norm;
+    if (SRC > 0) norm.request(p, wave, lane);
+    Group ga, gb;
+    (void) gb;
+    if (mine > 0) load(ga, 0);                             // the first weights are on their way while the activations are made
+    if (SRC != 0) {
         const int ldl = p.K + EPL;
         T * rows = (T *) (smem + 8 * NT * RM * 1024);
-        add_norm_prologue<T, TP ? TP : 1>(p, rows, ldl, red);
-        arow[0] = rows + (lr < p.T ? lr : p.T - 1) * ldl + g * EPL;
-    } else {
-#pragma unroll
-        for (int n = 0; n < NT; ++n) { const int t = t0 + n * 16 + lr; arow[n] = (const T *) p.act + (size_t) (t < p.T ? t : p.T - 1) * p.lda + g * EPL; }
+        if (SRC > 0) norm.finish(p, rows, ldl, red, wave, lane);
+        else {
+            const int n16 = p.K / EPL;
+            for (int t = 0; t < p.T; ++t)
+                for (int i = threadIdx.x; i < n16; i += 512) *(u32x4 *) (rows + t * ldl + i * EPL) = *(const PM_G u32x4 *) ((const T *) p.act + (size_t) t * p.lda + i * EPL);
+            __syncthreads();
+        }
+        const int t = lr % TOK;
+        arow[0] = rows + (t < p.T ? t : p.T - 1) * ldl + koff;
     }
     f32x4 acc[NT][RM];
 #pragma unroll
     for (int n = 0; n < NT; ++n)
 #pragma unroll
         for (int m = 0; m < RM; ++m) acc[n][m] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-    auto mma = [&](const u32x4 (&w)[U][RM][PB], int grp, bool full) __attribute__((always_inline)) {
+    auto mma = [&](const Group & a, int grp, bool full) __attribute__((always_inline)) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const int i = grp * U + u, k = (wave + i * 8) << 6;
@@ -122,55 +160,60 @@ template <typename T, int NT, int RM, int TP> __global__ __launch_bounds__(512) 
             for (int s = 0; s < PB; ++s)
 #pragma unroll
                 for (int n = 0; n < NT; ++n) {
-                    const u32x4 b = TP ? *(const u32x4 *) (arow[n] + k + s * (64 / PB)) : *(const PM_G u32x4 *) (arow[n] + k + s * (64 / PB));
+                    u32x4 x;
+                    if (NB) x = a.x[u][n][s]; else x = *(const u32x4 *) (arow[n] + k + s * (64 / PB));
 #pragma unroll
-                    for (int m = 0; m < RM; ++m) acc[n][m] = Frag<T>::mma(w[u][m][s], b, acc[n][m]);
+                    for (int m = 0; m < RM; ++m) acc[n][m] = Frag<T>::mma(a.w[u][m][s], x, acc[n][m]);
                 }
         }
     };
     // two register sets, the next group's loads in front of this group's products
     const int ng = (mine + U - 1) / U;
-    int g2 = 0;
-    for (; g2 + 2 < ng; g2 += 2) { load(wb, g2 + 1); mma(wa, g2, true); load(wa, g2 + 2); mma(wb, g2 + 1, true); }
-    if (ng - g2 == 2) { load(wb, g2 + 1); mma(wa, g2, true); mma(wb, g2 + 1, false); }
-    else if (ng - g2 == 1) mma(wa, g2, false);
+    int i = 0;
+    if (!TWO) for (; i < ng; ++i) { if (i) load(ga, i); mma(ga, i, false); }
+    else for (; i + 2 < ng; i += 2) { load(gb, i + 1); mma(ga, i, true); load(ga, i + 2); mma(gb, i + 1, true); }
+    if (TWO && ng - i == 2) { load(gb, i + 1); mma(ga, i, true); mma(gb, i + 1, false); }
+    else if (TWO && ng - i == 1) mma(ga, i, false);
 #pragma unroll
     for (int n = 0; n < NT; ++n)
 #pragma unroll
         for (int m = 0; m < RM; ++m) *(f32x4 *) (red + (((wave * NT + n) * RM + m) * 16 + lr) * 16 + g * 4) = acc[n][m];
     __syncthreads();
-    for (int o = threadIdx.x; o < NT * RM * 256; o += 512) {
-        const int r = o & 15, m = (o >> 4) % RM, t = (o >> 4) / RM;                     // rows fastest: a token's rows are stored as one segment
-        const int n = t >> 4, tt = t & 15;
+    for (int o = threadIdx.x; o < NT * RM * ROWS * TOK; o += 512) {
+        const int r = o % ROWS, m = o / ROWS % RM, t = o / ROWS / RM, n = t / TOK, tt = t % TOK;      // rows fastest: a token's rows are stored as one segment
+        const int row = r0 + m * ROWS + r, tok = t0 + t;
+        if (row >= p.n_store || tok >= p.T) continue;
         float v = 0.0f;
 #pragma unroll
-        for (int w = 0; w < 8; ++w) v += red[(((w * NT + n) * RM + m) * 16 + tt) * 16 + r];
-        const int row = r0 + m * 16 + r, tok = t0 + t;
-        if (row < p.n_store && tok < p.T) {
-            if (p.bias) v += p.bias[row];
-            if (p.act_fn == PM355_ACT_RELU2) { v = fmaxf(v, 0.0f); v *= v; }
-            st_type(p.y, (size_t) tok * p.ldy + row, p.y_type, v);
+        for (int w = 0; w < 8; ++w) {
+            const float * q = red + (((w * NT + n) * RM + m) * 16 + tt) * 16 + r;
+            v += q[0];
+            if (LINE) v += q[8 * 16 + 8];
         }
+        if (p.bias) v += p.bias[row];
+        if (p.act_fn == PM355_ACT_RELU2) { v = fmaxf(v, 0.0f); v *= v; }
+        st_type(p.y, (size_t) tok * p.ldy + row, p.y_type, v);
     }
 }
 
-template <typename T, int NT, int RM, int TP> int launch(const SmallP & p, int N, hipStream_t st) {
-    const size_t lds = (size_t) 8 * NT * RM * 1024 + (TP ? (size_t) p.T * (p.K * sizeof(T) + 16) : 0);
-    pm_allow_big_lds((const void *) dense_small_kernel<T, NT, RM, TP>, lds);
-    hipLaunchKernelGGL((dense_small_kernel<T, NT, RM, TP>), dim3(N / (16 * RM), (p.T + 16 * NT - 1) / (16 * NT)), dim3(512), lds, st, p);
+template <typename T, int NT, int RM, int SRC> int launch(const SmallP & p, int N, hipStream_t st) {
+    constexpr bool LINE = sizeof(T) == 2 && SRC != 0;
+    constexpr int rows = (LINE ? 8 : 16) * RM, toks = (LINE ? 8 : 16) * NT;
+    const size_t lds = (size_t) 8 * NT * RM * 1024 + (SRC ? (size_t) p.T * (p.K * sizeof(T) + 16) : 0);
+    pm_allow_big_lds((const void *) dense_small_kernel<T, NT, RM, SRC>, lds);
+    hipLaunchKernelGGL((dense_small_kernel<T, NT, RM, SRC>), dim3(N / rows, (p.T + toks - 1) / toks), dim3(512), lds, st, p);
     return 0;
 }
 template <typename T> int launch_type(const pm_dense_args & a, const SmallP & p, hipStream_t st) {
-    const int N = (a.n_store + 63) / 64 * 64;
+    const int N = (a.n_store + 63) / 64 * 64, per_wave = (a.K / 64 + 7) / 8;
+    const int rm = per_wave >= 8 ? 1 : 2;                  // (a wave's load group should not outgrow its share of K)
     if (a.pro) {
-        // every workgroup runs the prologue: few enough of them that all are resident (two per CU)
         if (!pm_dense_pro_ok(a.T, a.pro->width)) return PM355_E_UNSUPPORTED;
-        auto go = [&](auto rm) {
-            constexpr int RM = decltype(rm)::value;
-            return a.T == 1 ? launch<T, 1, RM, 1>(p, N, st) : a.T == 2 ? launch<T, 1, RM, 2>(p, N, st) : launch<T, 1, RM, 4>(p, N, st);
-        };
-        return N / 16 <= 512 ? go(std::integral_constant<int, 1>()) : N / 32 <= 512 ? go(std::integral_constant<int, 2>()) : go(std::integral_constant<int, 4>());
+        if constexpr (sizeof(T) == 2) if (rm == 2) return a.T == 1 ? launch<T, 1, 2, 1>(p, N, st) : a.T == 2 ? launch<T, 1, 2, 2>(p, N, st) : launch<T, 1, 2, 4>(p, N, st);
+        return a.T == 1 ? launch<T, 1, 1, 1>(p, N, st) : a.T == 2 ? launch<T, 1, 1, 2>(p, N, st) : launch<T, 1, 1, 4>(p, N, st);
     }
+    if constexpr (sizeof(T) == 2)
+        if (a.T <= 8 && (size_t) a.T * (a.K * 2 + 16) <= 72 * 1024) return rm == 1 ? launch<T, 1, 1, -1>(p, N, st) : launch<T, 1, 2, -1>(p, N, st);
     const bool wide = N / 32 >= 512;
     if (a.T <= 16) return wide ? launch<T, 1, 2, 0>(p, N, st) : launch<T, 1, 1, 0>(p, N, st);
     if (a.T <= 32) return wide ? launch<T, 2, 2, 0>(p, N, st) : launch<T, 2, 1, 0>(p, N, st);

@@ -34,6 +34,7 @@ CONFIGS = {
                    layer(heads=3, kv=3, dim=64, vdim=130, size=500, scale=0.4, cap=1.5, mix=False), width=136, vocab=75, eps=1e-3),
     "group": config(layer(heads=20, kv=1, dim=16, vdim=8, size=90), layer(heads=20, kv=1, dim=72, vdim=8, size=7, scale=0.3, cap=25.0), width=64, vocab=64),
     "huge_head": config(layer(heads=1, kv=1, dim=260, vdim=12, size=33, scale=0.06), layer(heads=2, kv=1, dim=8, vdim=12, size=1), width=40, vocab=33),
+    "late_mix": config(layer(mix=False, vdim=20), layer(vdim=24), layer(heads=3, kv=1, vdim=64, mix=False, ff=None), layer(heads=6, kv=2, dim=48, vdim=24, size=70, scale=0.5, cap=4.0)),
     "small": small_config(),
 }
 MODELS = {}
@@ -130,7 +131,7 @@ def test_dense_mul_mat_large_tiles(tiles):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("T,width", [(1, 96), (1, 2000), (2, 300), (3, 320), (4, 65)])
+@pytest.mark.parametrize("T,width", [(1, 96), (1, 2000), (2, 300), (2, 1024), (3, 320), (4, 65), (4, 512)])
 def test_norm_in_the_prologue_is_the_norm_launch(dtype, T, width):
     import prima_cpp_amd.ops as O
     K = (width + 63) // 64 * 64
@@ -148,6 +149,19 @@ def test_norm_in_the_prologue_is_the_norm_launch(dtype, T, width):
     y2 = torch.zeros(T, 128, device="cuda")
     O.dense_mul_mat(w, xb, y2)
     assert (y - y2).abs().max() <= (1e-5 if dtype == torch.float32 else 3e-2) * y2.abs().max()
+
+
+@pytest.mark.parametrize("rows,width", [(3, 70), (3, 1024), (2, 3000), (600, 3000), (2, 8192), (5, 9000)])
+def test_add_layer_norm(rows, width):
+    import prima_cpp_amd.ops as O
+    g = torch.Generator().manual_seed(width)
+    r, d = torch.randn(rows, width + 3, generator=g) * 2, torch.randn(rows, width + 3, generator=g) * 9 + 4
+    nw, nb = torch.randn(width, generator=g), torch.randn(width, generator=g)
+    want = r[:, :width].double().numpy() + P.layer_norm(d[:, :width].double().numpy(), nw.numpy(), nb.numpy(), 1e-3)
+    rd, xb = r.cuda(), torch.zeros(rows, width + 3, dtype=torch.bfloat16, device="cuda")
+    O.add_layer_norm(rd, d.cuda(), nw.cuda(), nb.cuda(), 1e-3, width, xb)
+    assert np.abs(rd[:, :width].cpu().numpy() - want).max() < 1e-5 * np.abs(want).max()
+    assert (rd[:, :width].bfloat16() == xb[:, :width]).all() and (rd[:, width:].cpu() == r[:, width:]).all() and (xb[:, width:] == 0).all()
 
 
 # ---- mechanisms ----------------------------------------------------------------------------------------------------------------------
