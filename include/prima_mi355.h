@@ -456,10 +456,14 @@ enum pm355_tensor_kind { PM355_T_ATTN_NORM = 0, PM355_T_WQ, PM355_T_WK, PM355_T_
                          PM355_T_TOK_EMBD, PM355_T_OUT_NORM, PM355_T_OUTPUT, PM355_T_ROPE_FREQS,
                          /* layer-described models; ATTN_NORM / FFN_NORM / OUT_NORM are the weights of the norms whose biases these are */
                          PM355_T_ATTN_NORM_B, PM355_T_FFN_NORM_B, PM355_T_OUT_NORM_B, PM355_T_W_OUT_GATE, PM355_T_SINK, PM355_T_VALUE_MIX, PM355_T_FFN_UP_B,
-                         PM355_T_FFN_DOWN_B, PM355_T_COUNT };
+                         PM355_T_FFN_DOWN_B,
+                         /* norms in front of a sublayer; bigram embedding; latent attention; selective scan; experts (part = expert) */
+                         PM355_T_ATTN_PRE_NORM, PM355_T_FFN_PRE_NORM, PM355_T_BIGRAM, PM355_T_DQ, PM355_T_DQ_NORM, PM355_T_UQ, PM355_T_DKV, PM355_T_DKV_NORM, PM355_T_UK, PM355_T_UV,
+                         PM355_T_SSM_IN, PM355_T_SSM_CONV, PM355_T_SSM_CONV_B, PM355_T_SSM_X, PM355_T_SSM_DT, PM355_T_SSM_DT_B, PM355_T_SSM_A_LOG, PM355_T_SSM_D, PM355_T_ROUTER,
+                         PM355_T_EXP_UP, PM355_T_EXP_DOWN, PM355_T_COUNT };
 enum { PM355_HAS_EMBD = 1, PM355_HAS_HEAD = 2 };
 
-/* Architectures are looked up by name ("llama", "qwen2", "kudirax"): the id for pm355_hparams.arch / pm355_stack_desc.arch, or PM355_E_UNSUPPORTED where this build
+/* Architectures are looked up by name ("llama", "qwen2", "kudirax", "keranex"): the id for pm355_hparams.arch / pm355_stack_desc.arch, or PM355_E_UNSUPPORTED where this build
  * does not carry the implementation. */
 PM355_API int pm355_arch_id(const char * name);
 
@@ -471,20 +475,33 @@ enum { PM355_MIX_QK_NORM    = 1,        /* q and k divided by their root mean sq
        PM355_MIX_SINK       = 2,        /* exp(sink[head]) joins the softmax denominator: no key, no value, neither scaled nor capped */
        PM355_MIX_VALUE_MIX  = 4,        /* v <- (1 - lambda) v + lambda v_first; v_first = v of the first layer with this flag, same token; the mix is what is cached */
        PM355_MIX_OUT_GATE   = 8 };      /* heads multiplied by sigmoid(W_g h) before the output projection */
-enum { PM355_MASK_CAUSAL = 0, PM355_MASK_CHUNK = 1 };      /* CHUNK: i sees j <= i with floor(i / size) == floor(j / size), counted from position 0 of the sequence */
-enum { PM355_FF_NONE = 0, PM355_FF_DENSE = 1 };            /* W_down act(W_up h + b_up) + b_down */
+enum { PM355_MASK_CAUSAL = 0, PM355_MASK_CHUNK = 1,        /* CHUNK: i sees j <= i with floor(i / size) == floor(j / size), counted from position 0 of the sequence */
+       PM355_MASK_WINDOW = 2 };                            /* i sees j with 0 <= i - j < size */
+/* Mixers. LATENT: queries W_uq norm(W_dq h), one cached row per token [norm(latent) | rotated key part] = W_dkv h, per-head keys W_uk c and values W_uv c; the rotated part of
+ * queries (per head) and key (shared) turns by position, pairs (i, i + rot_dims / 2). SSM: selective scan over a causal convolution of W_in h (mamba), state per sequence. */
+enum { PM355_MIXER_ATTENTION = 0, PM355_MIXER_LATENT = 1, PM355_MIXER_SSM = 2 };
+enum { PM355_FF_NONE = 0, PM355_FF_DENSE = 1,              /* W_down act(W_up h + b_up) + b_down */
+       PM355_FF_EXPERTS = 2 };                             /* sum over a token's n_expert_used experts of score * W_down act(W_up h); scores = softmax(W_router h), not renormalized,
+                                                              chosen among the n_group_keep groups (of n_group equal ones) with the largest single score */
 enum { PM355_ACT_NONE = 0, PM355_ACT_RELU2 = 1 };          /* square of relu */
 typedef struct {
     int32_t n_head, n_head_kv, k_dim, v_dim;   /* query head h reads KV head h / (n_head / n_head_kv) */
     int32_t mix_flags, mask, mask_size;
     float   scale, softcap;                    /* score = (q . k) * scale, then softcap * tanh(score / softcap) when softcap > 0 */
-    int32_t ff, n_ff, act;
+    int32_t ff, n_ff, act;                     /* n_ff: of one expert */
+    int32_t mixer;                             /* PM355_MIXER_*; LATENT: k_dim = unrotated size per head */
+    int32_t q_rank, kv_rank, rot_dim, rot_dims, kv_from; float rot_base;      /* LATENT; kv_from: layer whose cached rows this one reads, -1: its own */
+    int32_t inner, state, dt_rank, conv;       /* SSM */
+    int32_t n_expert, n_expert_used, n_group, n_group_keep;
 } pm355_layer_spec;
+enum { PM355_NORM_LAYER = 0, PM355_NORM_RMS = 1 };
 typedef struct {
     int32_t arch, n_layer, n_embd, n_vocab;
     int32_t type;                              /* PM355_TYPE_BF16: bf16 products with f32 accumulation; PM355_TYPE_F32: everything in 32-bit */
     float   norm_eps;
-    const pm355_layer_spec * layers;           /* n_layer of them; norms are layer norms with weight and bias on each sublayer's OUTPUT: x + norm(sublayer(x)) */
+    const pm355_layer_spec * layers;           /* n_layer of them; every sublayer's OUTPUT is normed: x + norm(sublayer(x)), with pre_norm x + norm(sublayer(pre_norm(x))) */
+    int32_t norm, pre_norm;                    /* PM355_NORM_*: LAYER has weight and bias, RMS a weight; pre_norm needs RMS */
+    int64_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;      /* buckets > 0: + bigram[(previous token * mul_prev + token * mul_cur) mod buckets], first token: row buckets */
 } pm355_stack_desc;
 PM355_API pm355_model * pm355_model_new_stack(const pm355_stack_desc * d);
 
@@ -525,6 +542,8 @@ PM355_API const char * pm355_model_error(pm355_model * m);
  * pinned double buffers (hipMemcpyAsync) and re-ordered into the HBM layout on the device
  * (replaces load_all_data's synchronous upload, src/llama.cpp:5418-5640). layer = -1 for per-model tensors. */
 PM355_API int pm355_model_set_tensor(pm355_model * m, int kind, int layer, int type, const void * host_data, size_t nbytes);
+/* one part of a tensor that comes in parts (PM355_T_EXP_*: part = expert); other tensors are their part 0 */
+PM355_API int pm355_model_set_tensor_part(pm355_model * m, int kind, int layer, int part, int type, const void * host_data, size_t nbytes);
 /* WINDOW STREAMING for windows larger than HBM (call before the first layer tensor is set): the layer tensors are kept in pinned
  * host memory (already in the HBM layout) and cycled through n_slots device-side layer slots by a copy stream (hipMemcpyAsync),
  * one layer ahead per free slot, while the compute stream works on the current layer - replaces prima.cpp's mmap prefetch /

@@ -20,7 +20,7 @@ LIB = os.path.join(HERE, "libprima_mi355.so")
 DENSE_LIB = os.path.join(HERE, "libprima_mi355_dense.so")
 PROBE_LIB = os.path.join(HERE, "libprima_mi355_probe.so")
 # what a layer-described (dense-weight) model needs: also a library of its own, so that such a model can be served without compiling the quantized kernels
-DENSE_SOURCES = ["c_api_base.hip", "model.hip", "kv_pool.hip", "stack.hip", "dense_small.hip", "dense_gemm.hip", "dense_ops.hip", "dense_api.hip", "attn_paged.hip", "repack.hip", "upload.hip"]
+DENSE_SOURCES = ["c_api_base.hip", "model.hip", "kv_pool.hip", "stack.hip", "dense_small.hip", "dense_gemm.hip", "dense_ops.hip", "dense_api.hip", "attn_paged.hip", "attn_latent.hip", "ssm.hip", "moe.hip", "repack.hip", "upload.hip"]
 SOURCES = DENSE_SOURCES + ["c_api.hip", "quantize.hip", "mmvq.hip", "mmvq_cols.hip", "layer_ops.hip", "ggml_ops.hip", "engine.hip", "mmq.hip", "mmq_pf.hip", "mmq_i8.hip", "mmq_big.hip",
            "attn_prefill.hip", "attn_cached.hip", "attn_flash_mfma.hip", "attn_split.hip", "attn_flash.hip", "attn_q8.hip", "ring.hip", "ts.hip"]
 # round 5's measured-slower forms of the decode layer (sum-of-squares partials, attention tail, persistent engine): a library of their own, loaded by their tests

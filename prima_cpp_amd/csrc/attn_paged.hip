@@ -1,4 +1,4 @@
-// attn_paged.hip — attention over paged KV caches: unit-norm q / k, capped scores, chunk masks, softmax with a sink, mixed values, output gate - each one a parameter
+// attn_paged.hip — attention over paged KV caches: unit-norm q / k, capped scores, chunk and window masks, softmax with a sink, mixed values, output gate - each one a parameter
 // (pm_attn_layer). Pages hold 64 tokens of one sequence per KV head: K rows [64][dkp], V transposed [dvp][64], so that both products read their matrix-core operands as
 // 16-byte pieces. Four kernels:
 //   prepare   q / k unit norm, value mixing, K / V into the pages (prompts; decode fuses it)
@@ -317,7 +317,7 @@ template <int DK, int DV, bool FIXED> __global__ __launch_bounds__(256, 2) void 
     tile = n_tiles - 1 - tile;                             // (the longest ones first)
     const pm_attn_tile tl = tiles[tile];
     const int g = h / (a.H / a.G);
-    const int32_t * pages = b.table + (size_t) tl.seq * b.table_ld;
+    const int32_t * pages = b.table + (a.flat ? 0 : (size_t) tl.seq * b.table_ld);
     const int qi = wave * 32 + lr, qc = qi < tl.n ? qi : tl.n - 1;
     const int pos = tl.pos + qc, first = first_key(pos, a.mask, a.mask_size);
     const int w_on = wave * 32 < tl.n, w_q1 = (wave * 32 + 31 < tl.n ? wave * 32 + 31 : tl.n - 1);
@@ -333,12 +333,12 @@ template <int DK, int DV, bool FIXED> __global__ __launch_bounds__(256, 2) void 
     // DMA: a page is K pieces then V pieces of 1 KiB; wave w brings pieces w, w + 4, ..
     const uint32_t lds0 = (uint32_t) (uintptr_t) (__attribute__((address_space(3))) char *) smem;
     auto request = [&](int pg, int stage) __attribute__((always_inline)) {
-        const size_t at = (size_t) __builtin_amdgcn_readfirstlane(pages[pg]) * a.G + g;
+        const size_t at = (size_t) __builtin_amdgcn_readfirstlane(a.flat ? tl.seq + pg : pages[pg]) * a.G + g;
         const char * kb = (const char *) a.kc + at * KB, * vb = (const char *) a.vc + at * (128 * DV);
 #pragma unroll
         for (int i = 0; i < DK / 32; ++i) {
             const uint32_t o = (uint32_t) (wave + i * 4) * 1024u + (uint32_t) lane * 16u, row = o / (DK * 2), ch = o % (DK * 2) / 16;
-            pm_dma16(kb, row * (DK * 2) + (ch ^ (DK == 64 ? (row >> 1) & 7 : row & 15)) * 16, lds0 + stage * STAGE + (wave + i * 4) * 1024);
+            pm_dma16(kb, row * (DK * 2) + (ch ^ (DK % 128 ? (row >> 1) & 7 : row & 15)) * 16, lds0 + stage * STAGE + (wave + i * 4) * 1024);
         }
 #pragma unroll
         for (int i = 0; i < DV / 32; ++i) {
@@ -370,7 +370,7 @@ template <int DK, int DV, bool FIXED> __global__ __launch_bounds__(256, 2) void 
         for (int t = 0; t < 2; ++t)
 #pragma unroll
             for (int e = 0; e < 16; ++e) s[t][e] = 0.0f;
-        const uint32_t sw = DK == 64 ? (kr >> 1) & 7 : kr & 15;
+        const uint32_t sw = DK % 128 ? (kr >> 1) & 7 : kr & 15;
 #pragma unroll
         for (int i = 0; i < KS; ++i)
 #pragma unroll
@@ -506,6 +506,7 @@ void pm_launch_attn_plain(const pm_attn_layer & a, const pm_batch_dev & b, int T
 int pm_launch_attn_tiles(const pm_attn_layer & a, const pm_batch_dev & b, const pm_attn_tile * d_tiles, int n_tiles, hipStream_t st) {
 #define PM_CALL(K, V) launch_tiles<K, V>(a, b, d_tiles, n_tiles, st)
     if (a.type != PM_BF16) return PM355_E_UNSUPPORTED;
+    if (a.dkp == 192 && a.dvp == 128) return PM_CALL(192, 128);
     PM_HEAD_SIZES(PM_CALL);
     return PM355_E_UNSUPPORTED;
 #undef PM_CALL

@@ -29,7 +29,7 @@ int pm355_dense_mul_mat_norm(int type, const void * W, int64_t K, int64_t N, con
     if (!W || !r || !d || !w || !b || !r_out || r_out == r || !y || K < 64 || width < 1 || width > K || ld < width || ldy < n_store || n_store < 1)
         return pm_api_fail(PM355_E_SHAPE, "dense_mul_mat_norm: shape", hipSuccess);
     (void) hipGetLastError();
-    const pm_add_norm pro{r, d, (int) ld, (int) ld, w, b, eps, width, r_out, (int) ld};
+    const pm_add_norm pro{r, d, (int) ld, (int) ld, w, b, eps, width, r_out, (int) ld, 0, nullptr, nullptr, 0};
     pm_dense_args a = dense_args(type, W, K, N, nullptr, 0, n_tokens, y, ldy, y_type, n_store, bias, act);
     a.pro = &pro;
     return done(pm_launch_dense(a, (hipStream_t) st), "dense_mul_mat_norm");
@@ -37,7 +37,7 @@ int pm355_dense_mul_mat_norm(int type, const void * W, int64_t K, int64_t N, con
 int pm355_add_layer_norm(int type, float * r, const float * d, int64_t ld, const float * w, const float * b, float eps, int width, int n_rows, void * xb, pm355_stream_t st) {
     if (!r || !d || !w || !b || width < 1 || width > 32768 || ld < width || n_rows < 1) return pm_api_fail(PM355_E_SHAPE, "add_layer_norm: shape", hipSuccess);
     (void) hipGetLastError();
-    pm_launch_add_layer_norm(type, r, d, (int) ld, (int) ld, w, b, eps, width, n_rows, xb, (hipStream_t) st);
+    pm_launch_add_norm(type, pm_norm_args{0, w, b, nullptr, eps, width, PM_F32, 0}, r, d, (int) ld, (int) ld, n_rows, xb, (int) ld, (hipStream_t) st);
     return done(0, "add_layer_norm");
 }
 size_t pm355_attn_paged_scratch(int n_tokens, int n_head, int n_head_kv, int v_pad) { return pm_attn_decode_part_floats(n_tokens, n_head_kv, n_head, v_pad); }

@@ -3,6 +3,7 @@
 // c ^ ((r >> 1) & 7): the sixteen lanes a ds_read_b128 serves hit sixteen bank groups). One barrier per stage: behind it the stage of the previous step is free and takes
 // the next k-step's DMA, which has this step's MFMAs to land. Tiles 256 x 256 (eight waves, 128 tokens x 64 rows each) or 128 x 128 (four waves, 64 x 64), chosen by how
 // many rounds the grid takes; tiles of one XCD form compact blocks of the output so that its L2 serves both operands.
+// The same loop multiplies experts (token tiles from the routing tables, rows gathered and scattered by pair) and expands latent cache pages into keys and transposed values.
 #include "pm355_dense.h"
 #include "pm355_kernels.h"
 #include "../../include/prima_mi355.h"
@@ -10,39 +11,63 @@
 
 namespace {
 
+enum { DENSE = 0, EXPERTS = 1, KEYS = 2, VALUES = 3 };
 struct GemmP {
     const uint16_t * W; const uint16_t * X; void * y; const float * bias;
     int K, N, T, lda, ldy, y_type, n_store, act_fn, nt, nn;      // nt, nn: token / row tiles
+    // EXPERTS: tiles = [count, {expert, first sorted pair, pairs} ..]; input rows are tokens (gather) or sorted pairs, output rows sorted pairs or pairs (scatter)
+    const int32_t * tiles, * order; const float * weight; int64_t e_stride; int top, gather, scatter;
+    // KEYS: X rows are those of cache pages; VALUES: the rows of W are (tokens become the columns of the output)
+    const int32_t * pages; int H, per, rows_h, pad;              // heads, values per head, rows of W per head, padded head size of the output
 };
 
-template <int BM, int BN, int WM, int WN> __global__ __launch_bounds__(BM / WM * (BN / WN) * 64) void dense_gemm_kernel(GemmP p) {
+template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__(BM / WM * (BN / WN) * 64) void dense_gemm_kernel(GemmP p) {
     constexpr int WAVES = BM / WM * (BN / WN), MI = WM / 32, NI = WN / 32, PIECES = (BM + BN) / 8 / WAVES, STAGE = (BM + BN) * 128;
     extern __shared__ __attribute__((aligned(1024))) char smem[];
-    const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 31, h = lane >> 5;
+    const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 31, h_ = lane >> 5;
     const int wm = wave / (BN / WN), wn = wave % (BN / WN);
     // tile order: XCD x = blockIdx % 8 takes a contiguous run of tiles; runs walk blocks of 8 token tiles column by column
     const int total = p.nt * p.nn, per = (total + 7) / 8;
     const int slot = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if (slot >= total || (int) (blockIdx.x >> 3) >= per) return;
     const int band = slot / (8 * p.nn), left = p.nt - band * 8, bh = left < 8 ? left : 8, in = slot - band * 8 * p.nn;
-    const int t0 = (band * 8 + in % bh) * BM, n0 = (in / bh) * BN;
+    int t0 = (band * 8 + in % bh) * BM, n_tok = p.T;
+    const int n0 = (in / bh) * BN;
+    const uint16_t * W = p.W;
+    if constexpr (KIND == EXPERTS) {                       // t0, n_tok: sorted pairs of this tile
+        const int tile = band * 8 + in % bh;
+        if (tile >= __builtin_amdgcn_readfirstlane(ld_g(p.tiles))) return;
+        const int32_t * tt = p.tiles + 1 + 3 * tile;
+        W += (int64_t) __builtin_amdgcn_readfirstlane(ld_g(tt)) * p.e_stride;
+        t0 = __builtin_amdgcn_readfirstlane(ld_g(tt + 1)); n_tok = t0 + __builtin_amdgcn_readfirstlane(ld_g(tt + 2));
+    }
 
     // DMA pieces of this wave (8 rows of 128 bytes each): the first half of the waves brings the tokens, the second half the rows of W
     static_assert(BM == BN, "a wave's pieces belong to one operand");
     const bool tok = wave < WAVES / 2;
-    const char * base = tok ? (const char *) (p.X + (size_t) t0 * p.lda) : (const char *) (p.W + (size_t) n0 * p.K);
-    const int last = tok ? p.T - 1 - t0 : p.N - 1 - n0;
-    const uint32_t pitch = (uint32_t) (tok ? p.lda : p.K) * 2u;
+    const char * base = tok ? (const char *) (KIND == VALUES ? W + (size_t) t0 * p.K : p.X + (KIND == EXPERTS ? 0 : (size_t) t0 * p.lda)) : (const char *) (W + (size_t) n0 * p.K);
+    const int last = tok ? n_tok - 1 - t0 : p.N - 1 - n0;
+    const bool paged = KIND == KEYS ? tok : KIND == VALUES ? !tok : false;
+    const char * pbase[PIECES];                            // (paged: a piece's eight rows lie in one page)
+    (void) pbase;
+    const uint32_t pitch = (uint32_t) (tok && KIND != VALUES ? p.lda : p.K) * 2u;
     const uint32_t lds0 = (uint32_t) (uintptr_t) (__attribute__((address_space(3))) char *) smem + (uint32_t) wave * PIECES * 1024u;
     uint32_t off[PIECES];
 #pragma unroll
     for (int i = 0; i < PIECES; ++i) {
         const int r = (wave * PIECES + i) * 8 + (lane >> 3), rr = tok ? r : r - BM;
-        off[i] = (uint32_t) (rr < last ? rr : last) * pitch + (uint32_t) ((lane & 7) ^ ((r >> 1) & 7)) * 16u;
+        int row = rr < last ? rr : last;
+        if constexpr (KIND == EXPERTS) if (tok) { row += t0; if (p.gather) row = ld_g(p.order + row) / p.top; }
+        const uint32_t swz = (uint32_t) ((lane & 7) ^ ((r >> 1) & 7)) * 16u;
+        if (KIND >= KEYS && paged) {
+            const int at = (tok ? t0 : n0) + (wave * PIECES + i) * 8 - (tok ? 0 : BM), lim = (tok ? n_tok : p.N) - 8, a8 = at < lim ? at : lim;      // (whole pages: a multiple of 8)
+            pbase[i] = (const char *) p.X + ((size_t) __builtin_amdgcn_readfirstlane(ld_g(p.pages + a8 / PM_PAGE)) * PM_PAGE + a8 % PM_PAGE) * (size_t) p.lda * 2;
+            off[i] = (uint32_t) (lane >> 3) * (uint32_t) p.lda * 2u + swz;
+        } else off[i] = (uint32_t) row * pitch + swz;
     }
     auto request = [&](int k, int stage) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < PIECES; ++i) pm_dma16(base + (size_t) k * 128, off[i], lds0 + (uint32_t) stage * STAGE + (uint32_t) i * 1024u);
+        for (int i = 0; i < PIECES; ++i) pm_dma16((KIND >= KEYS && paged ? pbase[i] : base) + (size_t) k * 128, off[i], lds0 + (uint32_t) stage * STAGE + (uint32_t) i * 1024u);
     };
     f32x16 acc[MI][NI];
 #pragma unroll
@@ -68,9 +93,9 @@ template <int BM, int BN, int WM, int WN> __global__ __launch_bounds__(BM / WM *
         for (int j = 0; j < 4; ++j) {
             bf16x8 a[MI], b[NI];
 #pragma unroll
-            for (int n = 0; n < NI; ++n) b[n] = *(const bf16x8 *) (s + brow[n] + (uint32_t) (((j * 2 + h) ^ bsw[n]) * 16));
+            for (int n = 0; n < NI; ++n) b[n] = *(const bf16x8 *) (s + brow[n] + (uint32_t) (((j * 2 + h_) ^ bsw[n]) * 16));
 #pragma unroll
-            for (int m = 0; m < MI; ++m) a[m] = *(const bf16x8 *) (s + arow[m] + (uint32_t) (((j * 2 + h) ^ asw[m]) * 16));
+            for (int m = 0; m < MI; ++m) a[m] = *(const bf16x8 *) (s + arow[m] + (uint32_t) (((j * 2 + h_) ^ asw[m]) * 16));
 #pragma unroll
             for (int m = 0; m < MI; ++m)
 #pragma unroll
@@ -82,26 +107,55 @@ template <int BM, int BN, int WM, int WN> __global__ __launch_bounds__(BM / WM *
     for (int n = 0; n < NI; ++n) {
         const int col = n0 + wn * WN + n * 32 + lr;
         const bool ok = col < p.n_store;
+        if constexpr (KIND == KEYS) {                      // K[page][head][slot][pad]
+            const int h = col / p.per, d = col - h * p.per;
+#pragma unroll
+            for (int m = 0; m < MI; ++m)
+#pragma unroll
+                for (int e = 0; e < 16; ++e) {
+                    const int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
+                    if (ok && tok < p.T) ((uint16_t *) p.y)[(((size_t) (tok / PM_PAGE) * p.H + h) * PM_PAGE + tok % PM_PAGE) * p.pad + d] = f2bf(acc[m][n][e]);
+                }
+            continue;
+        }
+        if constexpr (KIND == VALUES) {                    // V[page][head][pad][slot]: rows of the tile are W's, columns the keys
+#pragma unroll
+            for (int m = 0; m < MI; ++m)
+#pragma unroll
+                for (int e = 0; e < 16; ++e) {
+                    const int row = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_, h = row / p.rows_h, d = row - h * p.rows_h;
+                    if (ok && row < p.T && d < p.per && h < p.H) ((uint16_t *) p.y)[(((size_t) (col / PM_PAGE) * p.H + h) * p.pad + d) * PM_PAGE + col % PM_PAGE] = f2bf(acc[m][n][e]);
+                }
+            continue;
+        }
         const float bias = (ok && p.bias) ? p.bias[col] : 0.0f;
 #pragma unroll
         for (int m = 0; m < MI; ++m)
 #pragma unroll
             for (int e = 0; e < 16; ++e) {
-                const int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h;
-                float v = acc[m][n][e] + bias;
-                if (p.act_fn == PM355_ACT_RELU2) { v = fmaxf(v, 0.0f); v *= v; }
-                if (ok && tok < p.T) st_type(p.y, (size_t) tok * p.ldy + col, p.y_type, v);
+                int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
+                float v = act_apply(p.act_fn, acc[m][n][e] + bias);
+                if (!ok || tok >= n_tok) continue;
+                if constexpr (KIND == EXPERTS) {
+                    if (p.weight || p.scatter) {
+                        const int pair = ld_g(p.order + tok);
+                        if (p.weight) v *= ld_g(p.weight + pair);
+                        if (p.scatter) tok = pair;
+                    }
+                }
+                st_type(p.y, (size_t) tok * p.ldy + col, p.y_type, v);
             }
     }
 }
 
-template <int BM, int BN, int WM, int WN> int launch(GemmP p, hipStream_t st) {
+template <int BM, int BN, int WM, int WN, int KIND> int launch(GemmP p, hipStream_t st) {
     constexpr int threads = BM / WM * (BN / WN) * 64;
-    p.nt = (p.T + BM - 1) / BM; p.nn = (p.n_store + BN - 1) / BN;
+    if (KIND != EXPERTS) p.nt = (p.T + BM - 1) / BM;
+    p.nn = (p.n_store + BN - 1) / BN;
     const size_t lds = (size_t) 2 * (BM + BN) * 128;
-    pm_allow_big_lds((const void *) dense_gemm_kernel<BM, BN, WM, WN>, lds);
+    pm_allow_big_lds((const void *) dense_gemm_kernel<BM, BN, WM, WN, KIND>, lds);
     const int per = (p.nt * p.nn + 7) / 8;
-    hipLaunchKernelGGL((dense_gemm_kernel<BM, BN, WM, WN>), dim3(per * 8), dim3(threads), lds, st, p);
+    hipLaunchKernelGGL((dense_gemm_kernel<BM, BN, WM, WN, KIND>), dim3(per * 8), dim3(threads), lds, st, p);
     return 0;
 }
 
@@ -117,9 +171,34 @@ int pm_launch_dense_gemm(const pm_dense_args & a, hipStream_t st) {
     // rounds of the grid x time of a tile: a 256-tile does four times a 128-tile's work on a whole CU in ~3.4x its time (two 128-tiles share a CU)
     const long big = (long) ((a.T + 255) / 256) * ((a.n_store + 255) / 256), small = (long) ((a.T + 127) / 128) * ((a.n_store + 127) / 128);
     const double cb = (double) ((big + 255) / 256) * 1.7, cs = (double) ((small + 511) / 512);
-    return cb <= cs ? launch<256, 256, 128, 64>(p, st) : launch<128, 128, 64, 64>(p, st);
+    return cb <= cs ? launch<256, 256, 128, 64, DENSE>(p, st) : launch<128, 128, 64, 64, DENSE>(p, st);
 }
 
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st) {
-    return a.pro || a.type != PM_BF16 || a.T <= 64 ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
+    return a.pro || a.group || a.type != PM_BF16 || a.T <= 64 ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
+}
+
+int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st) {
+    const int64_t pairs = (int64_t) a.T * a.r.top;
+    if (a.type != PM_BF16 || a.T < 1 || a.width_p % 64 || a.ffp % 64 || (int64_t) a.T * a.ldx * 2 >= 1ll << 32 || pairs * a.ffp * 2 >= 1ll << 32) return PM355_E_SHAPE;
+    GemmP p = {};
+    p.tiles = a.r.tiles; p.order = a.r.order; p.top = a.r.top;
+    p.nt = (int) (pairs / 128 + (a.r.E < pairs ? a.r.E : pairs));                  // (most tiles there can be: every expert's last one may be short)
+    p.W = (const uint16_t *) a.up; p.e_stride = a.up_stride; p.X = (const uint16_t *) a.x; p.lda = a.ldx; p.K = a.width_p; p.N = p.n_store = a.ffp; p.y = a.hid; p.ldy = a.ffp;
+    p.y_type = PM_BF16; p.act_fn = a.act_fn; p.gather = 1; p.weight = a.r.w;
+    launch<128, 128, 64, 64, EXPERTS>(p, st);
+    p.W = (const uint16_t *) a.down; p.e_stride = a.down_stride; p.X = (const uint16_t *) a.hid; p.lda = a.ffp; p.K = a.ffp; p.N = a.width_p; p.n_store = a.width; p.y = a.y; p.ldy = a.ldy;
+    p.y_type = a.y_type; p.act_fn = PM355_ACT_NONE; p.gather = 0; p.scatter = 1; p.weight = nullptr;
+    return launch<128, 128, 64, 64, EXPERTS>(p, st);
+}
+
+int pm_launch_latent_expand(const pm_latent_expand & x, hipStream_t st) {
+    if (x.n_pages < 1 || x.kvp % 64 || x.ld % 64) return PM355_E_SHAPE;
+    GemmP p = {};
+    p.pages = x.pages; p.X = (const uint16_t *) x.cache; p.lda = x.ld; p.K = x.kvp; p.H = x.H;
+    GemmP k = p;
+    k.W = (const uint16_t *) x.Wk; k.T = x.n_pages * PM_PAGE; k.n_store = x.H * x.dim; k.N = pm_dense_pad(k.n_store); k.y = x.K; k.per = x.dim; k.pad = x.dkp;
+    launch<128, 128, 64, 64, KEYS>(k, st);
+    p.W = (const uint16_t *) x.Wv; p.T = pm_dense_pad(x.H * x.vrows); p.N = p.n_store = x.n_pages * PM_PAGE; p.y = x.V; p.per = x.vdim; p.rows_h = x.vrows; p.pad = x.dvp;
+    return launch<128, 128, 64, 64, VALUES>(p, st);
 }

@@ -1,12 +1,18 @@
-// dense_ops.hip — what surrounds the matrix products of a layer-described model: weight conversion, embedding, layer norms (f32), greedy tokens.
+// dense_ops.hip — what surrounds the matrix products of a layer-described model: weight conversion, embeddings, norms (f32), rotation tables, greedy tokens.
 #include "pm355_dense.h"
 #include "pm355_kernels.h"
 #include "../../include/prima_mi355.h"
 
 namespace {
 
-__global__ void convert_kernel(int src_type, const void * src, int type, void * dst, int K, long n, int Kp) {
-    for (long i = (long) blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long) gridDim.x * blockDim.x) st_type(dst, (size_t) (i / K) * Kp + i % K, type, ld_any(src, i, src_type));
+__global__ void convert_kernel(int src_type, const void * src, int type, void * dst, int K, long n, int Kp, int group, int gstride, int transpose) {
+    for (long i = (long) blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long) gridDim.x * blockDim.x) {
+        const long r = i / K, k = i % K, g = group ? r / group : 0, in = group ? r - g * group : r;
+        st_type(dst, transpose ? (size_t) (g * gstride + k) * Kp + in : (size_t) (g * gstride + in) * Kp + k, type, ld_any(src, i, src_type));
+    }
+}
+__global__ void ssm_decay_kernel(float * a, long n) {
+    for (long i = (long) blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long) gridDim.x * blockDim.x) a[i] = -expf(a[i]) * 1.4426950408889634f;
 }
 
 __device__ __forceinline__ uint32_t hash32(uint64_t x) {
@@ -16,19 +22,6 @@ __device__ __forceinline__ uint32_t hash32(uint64_t x) {
 __global__ void fill_kernel(int type, void * dst, int K, long n, int Kp, uint64_t seed, float mean, float amp) {
     for (long i = (long) blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long) gridDim.x * blockDim.x)
         st_type(dst, (size_t) (i / K) * Kp + i % K, type, mean + amp * ((float) (hash32(seed * 0x9E3779B97F4A7C15ULL + (uint64_t) i) & 0xFFFFFF) / 8388608.0f - 1.0f));
-}
-
-// x[t] = embedding row (f32), xb[t] = the same in T; workgroup (0, 0) brings the device page tables up to date (their readers are later launches)
-__global__ void embed_kernel(int type, const void * embed, int Kp, int width, pm_batch_dev b, float * x, void * xb) {
-    const int t = blockIdx.x;
-    if (t == 0) for (int i = threadIdx.x; i < b.n_upd[0]; i += blockDim.x) b.table[b.upd[2 * i]] = b.upd[2 * i + 1];
-    int tok = b.tok[t];
-    if (tok < 0) tok = b.last[b.seq[t]];
-    for (int c = threadIdx.x; c < Kp; c += blockDim.x) {
-        const float v = c < width ? ld_any(embed, (size_t) tok * Kp + c, type) : 0.0f;
-        x[(size_t) t * Kp + c] = v;
-        if (xb) st_type(xb, (size_t) t * Kp + c, type, v);
-    }
 }
 
 __device__ __forceinline__ float block_sum(float v, float * red) {
@@ -42,42 +35,98 @@ __device__ __forceinline__ float block_sum(float v, float * red) {
     return s;
 }
 
-// one row per workgroup. RES: x[row] += layer_norm(y[row]) and out = the sum in T; else out[row] = layer_norm(x[rows[row]]) in T. VP > 0: the row and everything that joins
-// it are requested at once, VP values per lane; 0: any width, row in LDS
-template <bool RES, int NTH, int VP> __global__ __launch_bounds__(NTH) void layer_norm_kernel(int type, float * x, const float * y, int ldx, int ldy, const int32_t * rows, const float * w,
-                                                                                             const float * b, float eps, int width, void * out, int ldo) {
+// one token per workgroup; the first workgroups bring page tables, previous tokens and counters up to date (their readers are later launches; a portion's previous token
+// is read and replaced by the workgroup of its first token)
+__global__ __launch_bounds__(256) void embed_kernel(pm_embed_args a, pm_batch_dev b) {
+    __shared__ float red[4];
+    const int t = blockIdx.x;
+    if (t == 0) {
+        for (int i = threadIdx.x; i < b.n_upd[0]; i += 256) b.table[b.upd[2 * i]] = b.upd[2 * i + 1];
+        for (int i = threadIdx.x; i < a.n_clear; i += 256) a.clear[i] = 0;
+    }
+    auto token = [&](int r) { const int k = b.tok[r]; return k < 0 ? b.last[b.seq[r]] : k; };
+    const int tok = token(t);
+    int64_t row = -1;
+    if (a.bigram) {
+        const int i = b.idx[t], before = b.pos[t] == 0 ? -1 : i ? token(t - 1) : b.prev[b.seq[t]];
+        row = before < 0 ? a.buckets : (before * a.mul_prev + tok * a.mul_cur) % a.buckets;
+        __syncthreads();                                   // (every wave has read prev)
+        if (i == 0 && threadIdx.x == 0) b.prev[b.seq[t]] = token(t + b.left[t]);
+    }
+    float s = 0.0f;
+    for (int c = threadIdx.x; c < a.Kp; c += 256) {
+        float v = c < a.width ? ld_any(a.embed, (size_t) tok * a.Kp + c, a.type) : 0.0f;
+        if (row >= 0 && c < a.width) v += ld_any(a.bigram, (size_t) row * a.Kp + c, a.type);
+        a.x[(size_t) t * a.Kp + c] = v;
+        s = fmaf(v, v, s);
+        if (a.out && !a.w2) st_type(a.out, (size_t) t * a.Kp + c, a.type, v);
+    }
+    if (!a.out || !a.w2) return;
+    const float rs = 1.0f / sqrtf(block_sum(s, red) / (float) a.width + a.eps);
+    for (int c = threadIdx.x; c < a.Kp; c += 256) st_type(a.out, (size_t) t * a.Kp + c, a.type, c < a.width ? a.x[(size_t) t * a.Kp + c] * (rs * a.w2[c]) : 0.0f);
+}
+__global__ void rope_table_kernel(const int32_t * pos, float base, int dims, float * cs) {
+    const int half = dims / 2;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) {
+        double sn, cn;                                     // (once per token and step: far positions keep the angle's low bits)
+        sincos((double) pos[blockIdx.x] * pow((double) base, -2.0 * i / dims), &sn, &cn);
+        float * o = cs + ((size_t) blockIdx.x * half + i) * 2;
+        o[0] = (float) cn; o[1] = (float) sn;
+    }
+}
+
+// one row per workgroup. RES: x[row] += norm(y[row]) and out = the sum (or its RMS norm with weight w2) in T; else out[row] = norm(x[rows[row]]) in T. VP > 0: the row and
+// everything that joins it are requested at once, VP values per lane; 0: any width, row in LDS
+template <bool RES, int NTH, int VP> __global__ __launch_bounds__(NTH) void norm_kernel(int type, pm_norm_args q, float * x, const void * y, int ldx, int ldy, const int32_t * rows, void * out,
+                                                                                       int ldo) {
     extern __shared__ __attribute__((aligned(16))) float row[];
     __shared__ float red[NTH / 64];
     constexpr int N = VP ? VP : 1;
-    const int r = blockIdx.x;
-    const float * src = RES ? y + (size_t) r * ldy : x + (size_t) (rows ? rows[r] : r) * ldx;
-    float v[N], xv[N], wv[N], bv[N], s = 0.0f;
+    const int r = blockIdx.x, width = q.width;
+    float * xr = x + (size_t) (!RES && rows ? rows[r] : r) * ldx;
+    auto value = [&](int c) __attribute__((always_inline)) -> float {        // what is normed
+        if (!RES) return ld_g(xr + c);
+        if (!q.parts) return q.y_type == PM_F32 ? ld_g((const float *) y + (size_t) r * ldy + c) : ld_any(y, (size_t) r * ldy + c, q.y_type);
+        float s = 0.0f;
+        for (int k = 0; k < q.parts; ++k) s += ld_any(y, ((size_t) r * q.parts + k) * ldy + c, q.y_type);
+        return s;
+    };
+    float v[N], xv[N], wv[N], bv[N], w2v[N], s = 0.0f;
     if (VP) {
 #pragma unroll
         for (int i = 0; i < N; ++i) {
             const int c = i * NTH + threadIdx.x, cc = c < width ? c : width - 1;
-            v[i] = ld_g(src + cc); wv[i] = ld_g(w + cc); bv[i] = ld_g(b + cc);
-            xv[i] = RES ? ld_g(x + (size_t) r * ldx + cc) : 0.0f;
+            v[i] = value(cc); wv[i] = ld_g(q.w + cc); bv[i] = q.b ? ld_g(q.b + cc) : 0.0f;
+            xv[i] = RES ? ld_g(xr + cc) : 0.0f;
+            w2v[i] = RES && q.w2 ? ld_g(q.w2 + cc) : 1.0f;
         }
 #pragma unroll
         for (int i = 0; i < N; ++i) s += i * NTH + (int) threadIdx.x < width ? v[i] : 0.0f;
-    } else for (int c = threadIdx.x; c < width; c += NTH) { const float f = src[c]; row[c] = f; s += f; }
-    const float mean = block_sum(s, red) / (float) width;
+    } else for (int c = threadIdx.x; c < width; c += NTH) { const float f = value(c); row[c] = f; s += f; }
+    const float mean = q.rms ? 0.0f : block_sum(s, red) / (float) width;
     float s2 = 0.0f;
     if (VP) {
 #pragma unroll
         for (int i = 0; i < N; ++i) { const float d = i * NTH + (int) threadIdx.x < width ? v[i] - mean : 0.0f; s2 = fmaf(d, d, s2); }
     } else for (int c = threadIdx.x; c < width; c += NTH) { const float d = row[c] - mean; s2 = fmaf(d, d, s2); }
-    const float rs = 1.0f / sqrtf(block_sum(s2, red) / (float) width + eps);
-    auto put = [&](int c, float f, float xo, float wo, float bo) __attribute__((always_inline)) {
+    const float rs = 1.0f / sqrtf(block_sum(s2, red) / (float) width + q.eps);
+    float s3 = 0.0f;
+    auto sum = [&](int c, float f, float xo, float wo, float bo) __attribute__((always_inline)) -> float {
         float o = (f - mean) * rs * wo + bo;
-        if (RES) { o = xo + o; x[(size_t) r * ldx + c] = o; }
-        if (out) st_type(out, (size_t) r * ldo + c, type, o);
+        if (RES) { o = xo + o; xr[c] = o; }
+        s3 = fmaf(o, o, s3);
+        return o;
     };
     if (VP) {
 #pragma unroll
-        for (int i = 0; i < N; ++i) { const int c = i * NTH + threadIdx.x; if (c < width) put(c, v[i], xv[i], wv[i], bv[i]); }
-    } else for (int c = threadIdx.x; c < width; c += NTH) put(c, row[c], RES ? x[(size_t) r * ldx + c] : 0.0f, w[c], b[c]);
+        for (int i = 0; i < N; ++i) { const int c = i * NTH + threadIdx.x; if (c < width) v[i] = sum(c, v[i], xv[i], wv[i], bv[i]); }
+    } else for (int c = threadIdx.x; c < width; c += NTH) row[c] = sum(c, row[c], RES ? xr[c] : 0.0f, q.w[c], q.b ? q.b[c] : 0.0f);
+    if (!out) return;
+    const float r2 = RES && q.w2 ? 1.0f / sqrtf(block_sum(s3, red) / (float) width + q.eps) : 1.0f;
+    if (VP) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) { const int c = i * NTH + threadIdx.x; if (c < width) st_type(out, (size_t) r * ldo + c, type, v[i] * (r2 * w2v[i])); }
+    } else for (int c = threadIdx.x; c < width; c += NTH) st_type(out, (size_t) r * ldo + c, type, row[c] * (r2 * (RES && q.w2 ? q.w2[c] : 1.0f)));
 }
 
 // index of the first maximum of every row (src/llama-sampling.cpp:390-397), also kept per sequence for the next step
@@ -102,35 +151,39 @@ __global__ __launch_bounds__(1024) void argmax_rows_kernel(const float * x, int 
 
 } // namespace
 
-void pm_launch_dense_convert(int src_type, const void * src, int type, void * dst, int K, int64_t N, int Kp, hipStream_t st) {
+void pm_launch_dense_convert(int src_type, const void * src, int type, void * dst, int K, int64_t N, int Kp, hipStream_t st, int group, int gstride, int transpose) {
     const long n = (long) N * K, g = (n + 255) / 256;
-    hipLaunchKernelGGL(convert_kernel, dim3((unsigned) (g < 65536 ? g : 65536)), dim3(256), 0, st, src_type, src, type, dst, K, n, Kp);
+    hipLaunchKernelGGL(convert_kernel, dim3((unsigned) (g < 65536 ? g : 65536)), dim3(256), 0, st, src_type, src, type, dst, K, n, Kp, group, gstride, transpose);
+}
+void pm_launch_ssm_decay(float * a, int64_t n, hipStream_t st) {
+    const long g = (n + 255) / 256;
+    hipLaunchKernelGGL(ssm_decay_kernel, dim3((unsigned) (g < 65536 ? g : 65536)), dim3(256), 0, st, a, (long) n);
 }
 void pm_launch_dense_fill(int type, void * dst, int K, int64_t N, int Kp, uint64_t seed, float mean, float amp, hipStream_t st) {
     const long n = (long) N * K, g = (n + 255) / 256;
     hipLaunchKernelGGL(fill_kernel, dim3((unsigned) (g < 65536 ? g : 65536)), dim3(256), 0, st, type, dst, K, n, Kp, seed, mean, amp);
 }
-void pm_launch_stack_embed(int type, const void * embed, int Kp, int width, const pm_batch_dev & b, int T, float * x, void * xb, hipStream_t st) {
-    hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, st, type, embed, Kp, width, b, x, xb);
+void pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st) { hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, st, a, b); }
+void pm_launch_rope_table(const int32_t * pos, int T, float base, int dims, float * cs, hipStream_t st) {
+    hipLaunchKernelGGL(rope_table_kernel, dim3(T), dim3(64), 0, st, pos, base, dims, cs);
 }
-template <bool RES> static void launch_norm(int type, float * x, const float * y, int ldx, int ldy, const int32_t * rows, const float * w, const float * b, float eps, int width, int n_rows,
-                                            void * out, int ldo, hipStream_t st) {
+template <bool RES> static void launch_norm(int type, const pm_norm_args & q, float * x, const void * y, int ldx, int ldy, const int32_t * rows, int n_rows, void * out, int ldo,
+                                            hipStream_t st) {
     auto go = [&](auto kern, int threads, size_t lds) {
         pm_allow_big_lds((const void *) kern, lds);
-        hipLaunchKernelGGL(kern, dim3(n_rows), dim3(threads), lds, st, type, x, y, ldx, ldy, rows, w, b, eps, width, out, ldo);
+        hipLaunchKernelGGL(kern, dim3(n_rows), dim3(threads), lds, st, type, q, x, y, ldx, ldy, rows, out, ldo);
     };
-    if (width <= 1024) go(layer_norm_kernel<RES, 256, 4>, 256, 0);
-    else if (width <= 4096 && n_rows > 512) go(layer_norm_kernel<RES, 256, 16>, 256, 0);
-    else if (width <= 4096) go(layer_norm_kernel<RES, 1024, 4>, 1024, 0);
-    else if (width <= 8192) go(layer_norm_kernel<RES, 1024, 8>, 1024, 0);
-    else go(layer_norm_kernel<RES, 1024, 0>, 1024, (size_t) width * 4);
+    if (q.width <= 1024) go(norm_kernel<RES, 256, 4>, 256, 0);
+    else if (q.width <= 4096 && n_rows > 512) go(norm_kernel<RES, 256, 16>, 256, 0);
+    else if (q.width <= 4096) go(norm_kernel<RES, 1024, 4>, 1024, 0);
+    else if (q.width <= 8192) go(norm_kernel<RES, 1024, 8>, 1024, 0);
+    else go(norm_kernel<RES, 1024, 0>, 1024, (size_t) q.width * 4);
 }
-void pm_launch_add_layer_norm(int type, float * x, const float * y, int ldx, int ldy, const float * w, const float * b, float eps, int width, int n_rows, void * xb, hipStream_t st) {
-    launch_norm<true>(type, x, y, ldx, ldy, nullptr, w, b, eps, width, n_rows, xb, ldx, st);
+void pm_launch_add_norm(int type, const pm_norm_args & q, float * x, const void * y, int ldx, int ldy, int n_rows, void * out, int ldo, hipStream_t st) {
+    launch_norm<true>(type, q, x, y, ldx, ldy, nullptr, n_rows, out, ldo, st);
 }
-void pm_launch_layer_norm_rows(int type, const float * x, int ldx, const int32_t * rows, const float * w, const float * b, float eps, int width, int n_rows, void * out, int ldo,
-                               hipStream_t st) {
-    launch_norm<false>(type, (float *) x, nullptr, ldx, 0, rows, w, b, eps, width, n_rows, out, ldo, st);
+void pm_launch_norm_rows(int type, const pm_norm_args & q, const float * x, int ldx, const int32_t * rows, int n_rows, void * out, int ldo, hipStream_t st) {
+    launch_norm<false>(type, q, (float *) x, nullptr, ldx, 0, rows, n_rows, out, ldo, st);
 }
 void pm_launch_argmax_rows(const float * logits, int n, int n_rows, int32_t * out, const int32_t * seq_of_row, int32_t * last, hipStream_t st) {
     hipLaunchKernelGGL(argmax_rows_kernel, dim3(n_rows), dim3(1024), 0, st, logits, n, out, seq_of_row, last);

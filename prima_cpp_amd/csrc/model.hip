@@ -28,6 +28,7 @@ void pm355_model_free(pm355_model * m) { delete m; }
 const char * pm355_model_error(pm355_model * m) { return m ? m->err : ""; }
 
 int pm355_model_set_tensor(pm355_model * m, int kind, int layer, int type, const void * host, size_t nbytes) { return m->set_tensor(kind, layer, type, host, nbytes); }
+int pm355_model_set_tensor_part(pm355_model * m, int kind, int layer, int part, int type, const void * host, size_t nbytes) { return m->set_tensor_part(kind, layer, part, type, host, nbytes); }
 int pm355_model_fill_tensor(pm355_model * m, int kind, int layer, int type, uint64_t seed, float scale) { return m->fill_tensor(kind, layer, type, seed, scale); }
 void * pm355_model_tensor_ptr(pm355_model * m, int kind, int layer, int * type_out) { return m->tensor_ptr(kind, layer, type_out); }
 int pm355_model_set_streaming(pm355_model * m, int n_slots) { return m ? m->set_streaming(n_slots) : PM355_E_SHAPE; }

@@ -12,10 +12,13 @@
 static inline int pm_dense_pad(int n) { return (n + 63) / 64 * 64; }
 static inline size_t pm_dense_bytes(int type) { return type == PM_BF16 ? 2 : 4; }
 
-// x + layer_norm(y) in the prologue of a mat-vec (few tokens): the normed sum is the activation row of every workgroup, workgroup 0 stores it as the new residual row
+// x + norm(y) in the prologue of a mat-vec (few tokens), where norm is a layer norm (weight, bias) or, with rms, y / sqrt(mean(y^2) + eps) * w; x == null: norm(y) alone. With
+// w2 the sum is RMS-normed once more on its way to the product (a norm in front of the sublayer). The result is the activation row of every workgroup; workgroup 0 stores
+// the sum as the new residual row (x_out) and the activations (act_out) where these are given
 struct pm_add_norm {
     const float * x; const float * y; int ldx, ldy; const float * w; const float * b; float eps; int width;
     float * x_out; int ldo;
+    int rms; const float * w2; void * act_out; int ld_act;
 };
 struct pm_dense_args {
     int type; const void * W; int K, N;                 // N: rows of W that exist (multiple of 64)
@@ -23,12 +26,17 @@ struct pm_dense_args {
     void * y; int ldy, y_type, n_store;                 // columns [0, n_store) of y are written
     const float * bias; int act_fn;                     // bias: n_store floats or null; act_fn: PM355_ACT_*
     const pm_add_norm * pro;                            // != null: the activations are x + norm(y) (pm_dense_pro_ok)
+    // group != 0 (a multiple of 32; the small-batch kernel, any T): one matrix per group of `group` rows (attention heads): group g multiplies the K activations from column
+    // g * g_act on, its first g_store rows go to the columns from g * g_out on
+    int group, g_act, g_out, g_store;
 };
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st);                    // picks the small-batch or the prompt kernel
 bool pm_dense_pro_ok(int T, int width);
 
-// f32 / bf16 host-order matrix [N][K] -> [rows at dst_row][Kp] of `type` (columns >= K stay as they are: zero from allocation)
-void pm_launch_dense_convert(int src_type, const void * src, int type, void * dst, int K, int64_t N, int Kp, hipStream_t st);
+// f32 / bf16 host-order matrix [N][K] -> [rows at dst_row][Kp] of `type` (columns >= K stay as they are: zero from allocation). group > 0: rows come in groups of `group`,
+// which start every `gstride` rows of dst; transpose: group g's rows become columns, dst row g * gstride + k
+void pm_launch_dense_convert(int src_type, const void * src, int type, void * dst, int K, int64_t N, int Kp, hipStream_t st, int group = 0, int gstride = 0, int transpose = 0);
+void pm_launch_ssm_decay(float * a, int64_t n, hipStream_t st);                  // a <- -exp(a) * log2(e)
 void pm_launch_dense_fill(int type, void * dst, int K, int64_t N, int Kp, uint64_t seed, float mean, float amp, hipStream_t st);
 
 // per-step tables of a batch in device memory (one upload per step): n tokens in the order of the entries
@@ -39,12 +47,26 @@ struct pm_batch_dev {
     const int32_t * last;           // [n_seq] last greedy token per sequence
     int32_t * table; int table_ld;  // [n_seq][table_ld] pool pages (device copy of the page tables)
     const int32_t * upd; const int32_t * n_upd;         // table updates of this step: pairs (index, page)
+    const int32_t * idx;            // [T] place of the token in its portion
+    const int32_t * left;           // [T] tokens of the portion behind it
+    int32_t * prev;                 // [n_seq] token in front of the portion (bigram embeddings), kept up to date by the embedding launch
 };
-void pm_launch_stack_embed(int type, const void * embed, int Kp, int width, const pm_batch_dev & b, int T, float * x, void * xb, hipStream_t st);
-// x += layer_norm(y) (y == null: x is normed in place of the sum: out = layer_norm(x)); xb = the same rows in T. rows: gather list or null
-void pm_launch_add_layer_norm(int type, float * x, const float * y, int ldx, int ldy, const float * w, const float * b, float eps, int width, int n_rows, void * xb, hipStream_t st);
-void pm_launch_layer_norm_rows(int type, const float * x, int ldx, const int32_t * rows, const float * w, const float * b, float eps, int width, int n_rows, void * out, int ldo,
-                               hipStream_t st);
+// what the embedding launch does: x = embed[token] + bigram[(previous token * mul_prev + token * mul_cur) mod buckets] (first token of a sequence: row `buckets`);
+// out = x, or its RMS norm with weight w2. It also brings page tables and `prev` up to date and clears `clear`
+struct pm_embed_args {
+    int type; const void * embed; int Kp, width;
+    const void * bigram; int64_t buckets, mul_prev, mul_cur;      // bigram null: none
+    const float * w2; float eps; int32_t * clear; int n_clear;
+    float * x; void * out;
+};
+void pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st);
+// x += norm(y); out = x (or, with w2, x / rms(x) * w2) in T. parts > 0: y is the sum of `parts` rows, y[row * parts ..]; y_type: of y
+struct pm_norm_args { int rms; const float * w, * b, * w2; float eps; int width; int y_type, parts; };
+void pm_launch_add_norm(int type, const pm_norm_args & n, float * x, const void * y, int ldx, int ldy, int n_rows, void * out, int ldo, hipStream_t st);
+// out[r] = norm(x[rows[r]]) in T (rows: gather list or null)
+void pm_launch_norm_rows(int type, const pm_norm_args & n, const float * x, int ldx, const int32_t * rows, int n_rows, void * out, int ldo, hipStream_t st);
+// cs[t][i] = cos, sin of pos[t] * base^(-2 i / dims), i < dims / 2
+void pm_launch_rope_table(const int32_t * pos, int T, float base, int dims, float * cs, hipStream_t st);
 void pm_launch_argmax_rows(const float * logits, int n, int n_rows, int32_t * out, const int32_t * seq_of_row, int32_t * last, hipStream_t st);
 
 // one attention layer over paged caches
@@ -58,6 +80,7 @@ struct pm_attn_layer {
     void * q;                               // [T][H][dkp] in T (written by pm_launch_attn_prepare)
     void * out; int ldo;                    // [T][H dv] in T (gate applied)
     float * part; unsigned * ticket; size_t part_floats;       // split-keys decode
+    int flat;                               // tiles kernel: a tile's page p is page seq + p of kc / vc (keys made for this step) instead of the sequence's pool page
 };
 // unit norm of q and k, value mixing, K / V into the pages
 void pm_launch_attn_prepare(const pm_attn_layer & a, const pm_batch_dev & b, int T, hipStream_t st);
@@ -70,6 +93,78 @@ int  pm_launch_attn_decode_paged(const pm_attn_layer & a, const pm_batch_dev & b
 void pm_launch_attn_plain(const pm_attn_layer & a, const pm_batch_dev & b, int T, hipStream_t st);
 size_t pm_attn_decode_part_floats(int n_tokens, int G, int H, int dvp);
 int  pm_attn_decode_splits(int n_tokens, int G, int max_keys);
+
+// one latent-attention layer (attn_latent.hip): keys and values of all heads are products of one cached row per token, [normed latent: kvp | rotated key part], ld values.
+// Decoded tokens attend in the latent itself (query and output matrices are applied to them instead of to every key); prompts expand the keys they see
+struct pm_latent_layer {
+    int type, H, dim, rot, rot_dims, kv_rank, kvp, ld; float scale, eps; int mask, mask_size;
+    void * cache;                           // [page][64][ld]
+    const void * raw; int ldraw, raw_type;  // projections [T][query latent: q_rank | latent: kv_rank | rot]
+    int q_rank; const float * q_norm; void * cq; int ld_cq;      // [T][ld_cq] normed query latent (written by pm_launch_latent_prepare)
+    const float * kv_norm;                  // null: the layer reads another layer's cache
+    void * qh; int qs;                      // [T][H][qs] queries, unrotated | rotated part
+    void * qa;                              // [T][H][ld] queries in the latent | rotated part
+    void * out; int ldo;                    // [T][ldo]: H x kvp weighted latents
+    const float * cs;                       // [T][rot_dims / 2][cos, sin]
+    float * part; unsigned * ticket; size_t part_floats;
+};
+// query latents normed (cq != null), latents normed and keys rotated into the cache (kv_norm != null)
+void pm_launch_latent_prepare(const pm_latent_layer & a, const pm_batch_dev & b, int T, hipStream_t st);
+// rotates the queries' rotated part: in place in qh, and into qa
+void pm_launch_latent_rotate(const pm_latent_layer & a, int T, hipStream_t st);
+// tokens 0 .. n - 1 of the step. fused: the cache store and the rotation of the queries happen inside (every entry is one token)
+int  pm_launch_latent_decode(const pm_latent_layer & a, const pm_batch_dev & b, int n, int fused, int max_keys, hipStream_t st);
+void pm_launch_latent_plain(const pm_latent_layer & a, const pm_batch_dev & b, int n, hipStream_t st);
+bool pm_latent_decode_ok(int kvp, int ld);
+size_t pm_latent_part_floats(int n_tokens, int H, int kvp);
+// keys of n_pages cache pages for the tiles kernel: K [page][H][64][dkp] (W_uk: [H * dim][kvp] plus the shared rotated part), V [page][H][dvp][64] (W_uv: per head vrows rows)
+struct pm_latent_expand { const void * cache; int ld, kvp; const int32_t * pages; int n_pages; const void * Wk, * Wv; int H, dim, rot, vdim, vrows; void * K, * V; int dkp, dvp; };
+int  pm_launch_latent_expand(const pm_latent_expand & e, hipStream_t st);       // the products
+void pm_launch_latent_spread(const pm_latent_expand & e, hipStream_t st);       // the rotated part, to every head
+
+// experts (moe.hip, dense_*.hip). Routing of T tokens: softmax over E logits, the `keep` best of `groups` groups of neighbours (by their largest score), the `top` largest
+// scores among these, not renormalized
+struct pm_route {
+    const float * logits; int ldl, E, top, groups, keep;
+    int32_t * id; float * w;                // [T * top] expert and weight per (token, slot)
+    int32_t * pos;                          // [T * top] place among the expert's pairs
+    int32_t * count;                        // [E] cleared by the embedding launch
+    int32_t * off;                          // [E + 1] first sorted pair of an expert
+    int32_t * order;                        // [T * top] sorted pairs
+    int32_t * active;                       // [1 + E] number of experts with pairs, and which
+    int32_t * tiles;                        // [1 + 3 n] number of 128-pair tiles, then {expert, first sorted pair, pairs} each
+};
+constexpr int PM_ROUTE_PAIR_MAX = 4, PM_ROUTE_ONE_MAX = 64;      // tokens up to which the pairs go one by one / one workgroup routes and sorts
+void pm_launch_route(const pm_route & r, int T, int want_tiles, hipStream_t st);
+struct pm_expert_args {
+    int type; pm_route r; int T, width_p, ffp, width;             // width_p, ffp: padded row lengths of up and down
+    const void * up, * down; int64_t up_stride, down_stride;      // values between experts: [E][ffp][width_p], [E][width_p][ffp]
+    int act_fn; const void * x; int ldx;                          // input rows in T
+    void * hid;                                                   // [T * top][ffp] in T: weight * act(W_up x)
+    void * y; int ldy, y_type;                                    // up to PM_ROUTE_PAIR_MAX tokens: [T] sums (f32); more: [T * top] rows, slot by slot
+};
+int pm_launch_experts_small(const pm_expert_args & a, hipStream_t st);
+int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st);
+
+// selective scan (ssm.hip): S[c, n] <- exp(dt A) S + dt x B, y = sum_n S C + D x, gated with silu(z); x: causal convolution + silu of the first half of the projections
+struct pm_scan_chunk { int32_t row, n, pos, seq, e_base, j, n_chunks, left; };      // up to 128 tokens of one portion; its place among the portion's chunks
+struct pm_ssm_layer {
+    int type, inner, innerp, state, sp, dt_rank, dtp, conv;       // sp: padded state (pm_ssm_state_pad)
+    const void * raw; int ldraw, raw_type;                        // [T][x: inner | z: inner]
+    const float * conv_w, * conv_b;                               // [inner][conv], [inner]
+    void * xc;                                                    // [T][innerp] in T
+    const void * f; int ldf;                                      // [T][dt: dtp | B: state | C: state] in T
+    const void * w_dt; const float * dt_b;                        // [innerp][dtp] in T
+    float * dt;                                                   // [T][innerp]: W_dt dt + bias, before the softplus (chunked scan)
+    const float * A2, * D;                                        // [inner][sp]: -exp(A_log) log2(e)
+    float * S, * cstate;                                          // [slot][inner][sp], [slot][conv - 1][innerp]
+    float * E, * dtsum;                                           // [chunk][inner][sp], [chunk][innerp]
+    void * y; int ldy;                                            // [T][ldy] in T
+};
+static inline int pm_ssm_state_pad(int n) { int p = 4; while (p < n) p *= 2; return p; }
+void pm_launch_ssm_conv(const pm_ssm_layer & a, const pm_batch_dev & b, int T, hipStream_t st);
+void pm_launch_ssm_step(const pm_ssm_layer & a, const pm_batch_dev & b, int T, hipStream_t st);      // every entry is one token: dt product, update, gate
+void pm_launch_ssm_scan(const pm_ssm_layer & a, const pm_batch_dev & b, const pm_scan_chunk * chunks, int n_chunks, int multi, hipStream_t st);
 
 #ifdef __HIPCC__
 #include "pm355_device.h"
@@ -105,5 +200,12 @@ __device__ __forceinline__ float cap_score(float s, float cap, float inv2cap_log
 }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + __expf(-z)); }
 // first key position the query at `pos` sees
-__device__ __forceinline__ int first_key(int pos, int mask, int size) { return mask == 1 ? pos - pos % size : 0; }
+__device__ __forceinline__ int first_key(int pos, int mask, int size) { return mask == 1 ? pos - pos % size : mask == 2 && pos >= size ? pos - size + 1 : 0; }
+__device__ __forceinline__ float silu32(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// activation functions of the dense products (PM355_ACT_*)
+__device__ __forceinline__ float act_apply(int fn, float v) {
+    if (fn == 1) { v = fmaxf(v, 0.0f); v *= v; }
+    return v;
+}
 #endif

@@ -11,6 +11,9 @@ struct pm355_model {
     virtual ~pm355_model() {}
 
     virtual int set_tensor(int kind, int layer, int type, const void * host, size_t nbytes) = 0;
+    virtual int set_tensor_part(int kind, int layer, int part, int type, const void * host, size_t nbytes) {      // part: expert
+        return part ? unsupported("set_tensor_part") : set_tensor(kind, layer, type, host, nbytes);
+    }
     virtual int fill_tensor(int kind, int layer, int type, uint64_t seed, float scale) = 0;
     virtual void * tensor_ptr(int, int, int *) { return nullptr; }
     virtual int set_streaming(int) { return unsupported("set_streaming"); }

@@ -11,7 +11,8 @@ from .lib import BF16, F32, Q4_K, Q5_K, Q6_K, Q8_0, check, ptr, stream_ptr  # no
 
 (T_ATTN_NORM, T_WQ, T_WK, T_WV, T_WO, T_FFN_NORM, T_FFN_GATE, T_FFN_UP, T_FFN_DOWN, T_BQ, T_BK, T_BV,
  T_TOK_EMBD, T_OUT_NORM, T_OUTPUT, T_ROPE_FREQS, T_ATTN_NORM_B, T_FFN_NORM_B, T_OUT_NORM_B, T_W_OUT_GATE, T_SINK, T_VALUE_MIX, T_FFN_UP_B,
- T_FFN_DOWN_B) = range(24)
+ T_FFN_DOWN_B, T_ATTN_PRE_NORM, T_FFN_PRE_NORM, T_BIGRAM, T_DQ, T_DQ_NORM, T_UQ, T_DKV, T_DKV_NORM, T_UK, T_UV, T_SSM_IN, T_SSM_CONV, T_SSM_CONV_B, T_SSM_X, T_SSM_DT, T_SSM_DT_B,
+ T_SSM_A_LOG, T_SSM_D, T_ROUTER, T_EXP_UP, T_EXP_DOWN) = range(45)
 HAS_EMBD, HAS_HEAD = 1, 2
 
 _vp, _i32, _i64, _sz = C.c_void_p, C.c_int, C.c_int64, C.c_size_t
@@ -29,18 +30,24 @@ class LayerSpec(C.Structure):
     """One layer of a layer-described model (pm355_layer_spec): sizes, mechanisms, constants."""
     _fields_ = [("n_head", C.c_int32), ("n_head_kv", C.c_int32), ("k_dim", C.c_int32), ("v_dim", C.c_int32),
                 ("mix_flags", C.c_int32), ("mask", C.c_int32), ("mask_size", C.c_int32), ("scale", C.c_float), ("softcap", C.c_float),
-                ("ff", C.c_int32), ("n_ff", C.c_int32), ("act", C.c_int32)]
+                ("ff", C.c_int32), ("n_ff", C.c_int32), ("act", C.c_int32), ("mixer", C.c_int32),
+                ("q_rank", C.c_int32), ("kv_rank", C.c_int32), ("rot_dim", C.c_int32), ("rot_dims", C.c_int32), ("kv_from", C.c_int32), ("rot_base", C.c_float),
+                ("inner", C.c_int32), ("state", C.c_int32), ("dt_rank", C.c_int32), ("conv", C.c_int32),
+                ("n_expert", C.c_int32), ("n_expert_used", C.c_int32), ("n_group", C.c_int32), ("n_group_keep", C.c_int32)]
 
 
 MIX_QK_NORM, MIX_SINK, MIX_VALUE_MIX, MIX_OUT_GATE = 1, 2, 4, 8
-MASK_CAUSAL, MASK_CHUNK = 0, 1
-FF_NONE, FF_DENSE = 0, 1
+MASK_CAUSAL, MASK_CHUNK, MASK_WINDOW = 0, 1, 2
+MIXER_ATTENTION, MIXER_LATENT, MIXER_SSM = 0, 1, 2
+FF_NONE, FF_DENSE, FF_EXPERTS = 0, 1, 2
+NORM_LAYER, NORM_RMS = 0, 1
 ACT_NONE, ACT_RELU2 = 0, 1
 
 
 class StackDesc(C.Structure):
     _fields_ = [("arch", C.c_int32), ("n_layer", C.c_int32), ("n_embd", C.c_int32), ("n_vocab", C.c_int32), ("type", C.c_int32),
-                ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec))]
+                ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec)), ("norm", C.c_int32), ("pre_norm", C.c_int32),
+                ("bigram_buckets", C.c_int64), ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64)]
 
 
 class BatchEntry(C.Structure):
@@ -89,6 +96,7 @@ def _lib():
             "pm355_model_free": (None, [_vp]),
             "pm355_model_error": (C.c_char_p, [_vp]),
             "pm355_model_set_tensor": (_i32, [_vp, _i32, _i32, _i32, _vp, _sz]),
+            "pm355_model_set_tensor_part": (_i32, [_vp, _i32, _i32, _i32, _i32, _vp, _sz]),
             "pm355_model_fill_tensor": (_i32, [_vp, _i32, _i32, _i32, C.c_uint64, C.c_float]),
             "pm355_model_finalize": (_i32, [_vp, _i32]),
             "pm355_model_finalize_seqs": (_i32, [_vp, _i32, _i32]),
@@ -146,10 +154,11 @@ class Model:
             pass
 
     # ---- tensors -----------------------------------------------------------------------------
-    def set_tensor(self, kind, layer, qtype, data):
+    def set_tensor(self, kind, layer, qtype, data, part=0):
+        """part: expert of T_EXP_UP / T_EXP_DOWN"""
         data = np.ascontiguousarray(data)
-        self._chk(self.lib.pm355_model_set_tensor(self.h, kind, layer, qtype, data.ctypes.data, data.nbytes),
-                  f"set_tensor(kind={kind}, layer={layer})")
+        self._chk(self.lib.pm355_model_set_tensor_part(self.h, kind, layer, part, qtype, data.ctypes.data, data.nbytes),
+                  f"set_tensor(kind={kind}, layer={layer}, part={part})")
 
     def fill_tensor(self, kind, layer, qtype, seed, scale):
         self._chk(self.lib.pm355_model_fill_tensor(self.h, kind, layer, qtype, seed, scale), "fill_tensor")
@@ -373,15 +382,16 @@ class Window(Model):
 
 
 class Stack(Model):
-    """A layer-described model with dense weights and a paged cache (pm355_model_new_stack). layers: LayerSpec list; type BF16 or F32."""
+    """A layer-described model with dense weights and a paged cache (pm355_model_new_stack). layers: LayerSpec list; type BF16 or F32; norm: NORM_* of the sublayers' outputs
+    and the head; pre_norm: RMS norms in front of the sublayers too; bigram: (buckets, mul_prev, mul_cur) or None."""
 
-    def __init__(self, arch, layers, n_embd, n_vocab, norm_eps, type=BF16):
+    def __init__(self, arch, layers, n_embd, n_vocab, norm_eps, type=BF16, norm=NORM_LAYER, pre_norm=False, bigram=None):
         self.lib = _lib()
         self.specs = (LayerSpec * len(layers))(*layers)
         aid = self.lib.pm355_arch_id(arch.encode())
         if aid < 0:
             raise L.PM355Error(f"architecture {arch} is not in this build")
-        self.desc = StackDesc(aid, len(layers), n_embd, n_vocab, type, norm_eps, self.specs)
+        self.desc = StackDesc(aid, len(layers), n_embd, n_vocab, type, norm_eps, self.specs, norm, int(pre_norm), *(bigram or (0, 0, 0)))
         self.h = self.lib.pm355_model_new_stack(C.byref(self.desc))
         if not self.h:
             raise L.PM355Error("pm355_model_new_stack failed (sizes out of range, or not enough memory)")
@@ -398,21 +408,30 @@ class Stack(Model):
 
     def fill_synthetic(self, seed=1234):
         """Random weights generated in HBM (bench)."""
-        E = self.desc.n_embd
+        E, bias, pre = self.desc.n_embd, self.desc.norm == NORM_LAYER, self.desc.pre_norm
         self.fill_tensor(T_TOK_EMBD, -1, self.type, seed + 1, 1.0)
         self.fill_tensor(T_OUTPUT, -1, self.type, seed + 2, 2.0 / np.sqrt(E))
         self.fill_tensor(T_OUT_NORM, -1, F32, seed + 3, 0.0)
-        self.fill_tensor(T_OUT_NORM_B, -1, F32, seed + 4, 0.1)
+        if bias:
+            self.fill_tensor(T_OUT_NORM_B, -1, F32, seed + 4, 0.1)
+        if self.desc.bigram_buckets:
+            self.fill_tensor(T_BIGRAM, -1, self.type, seed + 5, 0.5)
         for i, s in enumerate(self.specs):
             k = seed * 1000003 + i * 131
-            for j, (kind, width) in enumerate(((T_WQ, E), (T_WK, E), (T_WV, E), (T_WO, s.n_head * s.v_dim), (T_W_OUT_GATE, E if s.mix_flags & MIX_OUT_GATE else 0),
-                                               (T_FFN_UP, E if s.ff else 0), (T_FFN_DOWN, s.n_ff if s.ff else 0))):
+            att, lat, ssm, dense, moe = (s.mixer == MIXER_ATTENTION), (s.mixer == MIXER_LATENT), (s.mixer == MIXER_SSM), s.ff == FF_DENSE, s.ff == FF_EXPERTS
+            own = lat and s.kv_from < 0
+            for j, (kind, width) in enumerate(((T_WQ, E * att), (T_WK, E * att), (T_WV, E * att), (T_WO, s.inner if ssm else s.n_head * s.v_dim),
+                                               (T_W_OUT_GATE, E * att if s.mix_flags & MIX_OUT_GATE else 0), (T_FFN_UP, E * dense), (T_FFN_DOWN, s.n_ff * dense),
+                                               (T_DQ, E * lat), (T_UQ, s.q_rank * lat), (T_DKV, E * own), (T_UK, s.kv_rank * lat), (T_UV, s.kv_rank * lat), (T_SSM_IN, E * ssm),
+                                               (T_SSM_X, s.inner * ssm), (T_SSM_DT, s.dt_rank * ssm), (T_ROUTER, E * moe), (T_EXP_UP, E * moe), (T_EXP_DOWN, s.n_ff * moe))):
                 if width:
                     self.fill_tensor(kind, i, self.type, k + j, 2.0 / np.sqrt(width))
-            for j, (kind, on) in enumerate(((T_ATTN_NORM, 1), (T_ATTN_NORM_B, 1), (T_FFN_NORM, s.ff), (T_FFN_NORM_B, s.ff), (T_FFN_UP_B, s.ff), (T_FFN_DOWN_B, s.ff),
-                                            (T_SINK, s.mix_flags & MIX_SINK), (T_VALUE_MIX, s.mix_flags & MIX_VALUE_MIX))):
+            for j, (kind, on) in enumerate(((T_ATTN_NORM, 1), (T_ATTN_NORM_B, bias), (T_FFN_NORM, s.ff), (T_FFN_NORM_B, s.ff and bias), (T_FFN_UP_B, dense), (T_FFN_DOWN_B, dense),
+                                            (T_SINK, att and s.mix_flags & MIX_SINK), (T_VALUE_MIX, att and s.mix_flags & MIX_VALUE_MIX), (T_ATTN_PRE_NORM, pre),
+                                            (T_FFN_PRE_NORM, pre and s.ff), (T_DQ_NORM, lat), (T_DKV_NORM, own), (T_SSM_CONV, ssm), (T_SSM_CONV_B, ssm), (T_SSM_DT_B, ssm),
+                                            (T_SSM_A_LOG, ssm), (T_SSM_D, ssm))):
                 if on:
-                    self.fill_tensor(kind, i, F32, k + 50 + j, 0.1)
+                    self.fill_tensor(kind, i, F32, k + 50 + j, 0.5 if kind in (T_SSM_CONV, T_SSM_A_LOG) else 0.1)
 
 
 def smoke(oracle):

@@ -63,4 +63,4 @@ def _gguf_window(arch):
 register("llama")(_gguf_window(0))
 register("qwen2")(_gguf_window(1))
 
-from . import kudirax  # noqa: E402,F401  (registers itself)
+from . import keranex, kudirax  # noqa: E402,F401  (they register themselves)
