@@ -227,6 +227,17 @@ template <typename T, int NT, int RM, int SRC, int EXP> __global__ __launch_boun
     else for (; i + 2 < ng; i += 2) { load(gb, i + 1); mma(ga, i, true); load(ga, i + 2); mma(gb, i + 1, true); }
     if (TWO && ng - i == 2) { load(gb, i + 1); mma(ga, i, true); mma(gb, i + 1, false); }
     else if (TWO && ng - i == 1) mma(ga, i, false);
+    // A wave with nothing left to multiply comes here by a jump, and behind one of those jumps ROCm 7.2's compiler left out the wait states between a product and the store
+    // that reads it (seen in the assembly of the sorted-experts kernels, and in their results): they are spelled out. 20 states: the longest such wait there is
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int m = 0; m < RM; ++m) asm volatile("" : "+v"(acc[n][m]));
+    asm volatile("s_nop 15\n\ts_nop 3");
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int m = 0; m < RM; ++m) asm volatile("" : "+v"(acc[n][m]));
 #pragma unroll
     for (int n = 0; n < NT; ++n)
 #pragma unroll

@@ -152,8 +152,9 @@ def bf16(a):
     return ((u + 0x7FFF + ((u >> 16) & 1)) & np.uint32(0xFFFF0000)).view(np.float32)
 
 
-def random_model(cfg, seed):
-    """weights name -> float32 array of bfloat16 values, of a size at which every mechanism matters"""
+def random_model(cfg, seed, decisive=False):
+    """weights name -> float32 array of bfloat16 values, of a size at which every mechanism matters. decisive: a few entries of the residual stream tell the routers (and nobody
+    else) which class a token has, and no sublayer changes them, so that rounding cannot turn a choice of experts around"""
     rng = np.random.default_rng(seed)
     W, V, w = cfg["width"], cfg["vocab"], {}
 
@@ -200,4 +201,19 @@ def random_model(cfg, seed):
                 mat(p + "mlp.e%d.down" % e, W, F)
     vec("final.norm", W)
     mat("head", V, W, 2.0)
+    if decisive:
+        n, code = 5, slice(0, 5)
+        w["embed"][:, code] = 0.0
+        w["embed"][np.arange(V), np.arange(V) % n] = 0.5 * np.sqrt(W)
+        if b:
+            w["bigram"][:, code] = 0.0
+        w["head"][:, code] = 0.0
+        for k in w:
+            if k.endswith(("norm1b", "norm2b")):
+                w[k][code] = 0.0
+            elif k.endswith((".dq", ".dkv", "mix.in", ".up")):
+                w[k][:, code] = 0.0
+            elif k.endswith("router"):
+                w[k] *= 0.02
+                w[k][:, code] = np.stack([rng.permutation(np.linspace(-1, 1, len(w[k]))) for _ in range(n)], axis=1) * (0.5 * len(w[k]) / np.sqrt(W))
     return {k: bf16(v) for k, v in w.items()}
