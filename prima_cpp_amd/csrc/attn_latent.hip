@@ -119,8 +119,6 @@ template <typename T> __global__ __launch_bounds__(256) void plain_kernel(pm_lat
     }
 }
 
-__device__ __forceinline__ void st_shared(float * p, float v) { __hip_atomic_store((PM_G float *) p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
-__device__ __forceinline__ float ld_shared(const float * p) { return __hip_atomic_load((const PM_G float *) p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
 // waits until at most n of the wave's vector-memory operations are outstanding (rounded down to a count the instruction is spelled for)
 __device__ __forceinline__ void vm_wait(int n) {
     if (n >= 24) asm volatile("s_waitcnt vmcnt(24)" ::: "memory");
@@ -138,12 +136,12 @@ __device__ __forceinline__ void vm_wait(int n) {
 }
 
 // VT: 16-column value tiles per wave (kvp <= 128 VT). A wave's 16-byte pieces of the scores' k range and its DMA pieces per step are at most VT + 2
-template <int VT> __global__ __launch_bounds__(DW * 64) void latent_decode_kernel(pm_latent_layer a, pm_batch_dev b, int fused, int splits, int stages) {
+template <int VT> __global__ __launch_bounds__(DW * 64) void latent_decode_kernel(pm_latent_layer a, pm_batch_dev b, int fused, int splits, int stages,
+                                                                                                      float * ml) {
     constexpr int QS = VT + 2;
     extern __shared__ __attribute__((aligned(1024))) char smem[];
     const uint32_t pitch = (uint32_t) a.ld * 2u, stage_bytes = pitch * STEP;
     float * sp = (float *) (smem + stages * stage_bytes);  // [4 k ranges][2 key tiles][64 lanes][4]
-    __shared__ int is_last;
     const int h0 = blockIdx.y * 16, nh = a.H - h0 < 16 ? a.H - h0 : 16, t = blockIdx.x;
     const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 15, lg = lane >> 4;
     const int pos = __builtin_amdgcn_readfirstlane(ld_g(b.pos + t)), first = first_key(pos, a.mask, a.mask_size);
@@ -266,46 +264,40 @@ template <int VT> __global__ __launch_bounds__(DW * 64) void latent_decode_kerne
             }
         return;
     }
-    // partials out, then a ticket; the last split of this (token, 16 heads) merges all of them and re-arms the ticket
-    const size_t slot = (size_t) blockIdx.x * gridDim.y + blockIdx.y;
-    float * part = a.part + slot * splits * 16 * (a.kvp + 2);
+    const size_t slot = ((size_t) blockIdx.x * gridDim.y + blockIdx.y) * splits + s;
     if (lr < nh) {
-        float * r = part + (size_t) (s * 16 + lr) * (a.kvp + 2);
+        float * r = a.part + (slot * 16 + lr) * a.kvp + lg * 4;
 #pragma unroll
         for (int i = 0; i < VT; ++i) {
             const int dt = wave + i * DW;
-            if (dt < vt)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) st_shared(r + dt * 16 + lg * 4 + e, acc[i][e]);
+            if (dt < vt) *(PM_G f32x4 *) (r + dt * 16) = acc[i];
         }
-        if (wave == 0 && lg == 0) { st_shared(r + a.kvp, m); st_shared(r + a.kvp + 1, l); }
+        if (wave == 0 && lg == 0) *(PM_G u32x2 *) (ml + (slot * 16 + lr) * 2) = u32x2{__builtin_bit_cast(uint32_t, m), __builtin_bit_cast(uint32_t, l)};
     }
-    pm_vm_drain();
-    __syncthreads();
-    if (threadIdx.x == 0) {
-        unsigned * tk = a.ticket + slot;
-        is_last = __hip_atomic_fetch_add(tk, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (unsigned) splits - 1;
-        if (is_last) __hip_atomic_store(tk, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+// split sums of one (token, head) -> its weighted latent
+__global__ __launch_bounds__(256) void latent_merge_kernel(pm_latent_layer a, const float * ml, int splits) {
+    __shared__ float share[64];
+    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+    const size_t slot = ((size_t) t * ((a.H + 15) / 16) + h / 16) * splits;
+    if (threadIdx.x < 64) {
+        const float * q = ml + ((slot + (lane < splits ? lane : 0)) * 16 + h % 16) * 2;
+        const float m = lane < splits ? ld_g(q) : NONE, l = lane < splits ? ld_g(q + 1) : 0.0f, f = __builtin_amdgcn_exp2f(m - wave_max(m));
+        share[lane] = f / wave_sum(l * f);
     }
     __syncthreads();
-    if (!is_last) return;
-    float * ml = (float *) smem;                           // [splits][16][2]
-    for (int o = threadIdx.x; o < splits * 32; o += DW * 64) if ((o >> 1 & 15) < nh) ml[o] = ld_shared(part + (size_t) (o >> 1) * (a.kvp + 2) + a.kvp + (o & 1));
-    __syncthreads();
-    for (int h = 0; h < nh; ++h)
-        for (int d = threadIdx.x; d < a.kvp; d += DW * 64) {
-            float M = NONE, y = 0.0f, L = 0.0f;
-            for (int i = 0; i < splits; ++i) M = fmaxf(M, ml[(i * 16 + h) * 2]);
-            for (int i0 = 0; i0 < splits; i0 += 8) {
-                float r[8];
+    for (int d = threadIdx.x; d < a.kvp; d += 256) {
+        const float * r = a.part + (slot * 16 + h % 16) * a.kvp + d;
+        float y = 0.0f;
+        for (int i0 = 0; i0 < splits; i0 += 8) {
+            float v[8];
 #pragma unroll
-                for (int i = 0; i < 8; ++i) r[i] = ld_shared(part + (size_t) ((i0 + i < splits ? i0 + i : splits - 1) * 16 + h) * (a.kvp + 2) + d);
+            for (int i = 0; i < 8; ++i) v[i] = ld_g(r + (size_t) (i0 + i < splits ? i0 + i : 0) * 16 * a.kvp);
 #pragma unroll
-                for (int i = 0; i < 8; ++i)
-                    if (i0 + i < splits) { const float f = __builtin_amdgcn_exp2f(ml[((i0 + i) * 16 + h) * 2] - M); y += r[i] * f; L += ml[((i0 + i) * 16 + h) * 2 + 1] * f; }
-            }
-            ((uint16_t *) a.out)[(size_t) t * a.ldo + (size_t) (h0 + h) * a.kvp + d] = f2bf(y / L);
+            for (int i = 0; i < 8; ++i) y = fmaf(v[i], i0 + i < splits ? share[i0 + i] : 0.0f, y);
         }
+        ((uint16_t *) a.out)[(size_t) t * a.ldo + (size_t) h * a.kvp + d] = f2bf(y);
+    }
 }
 
 constexpr size_t LDS_MAX = 150 * 1024, SCORES = 8192;
@@ -335,12 +327,16 @@ void pm_launch_latent_plain(const pm_latent_layer & a, const pm_batch_dev & b, i
 }
 bool pm_latent_decode_ok(int kvp, int ld) { return kvp % 64 == 0 && ld % 64 == 0 && ld >= kvp && kvp <= 1024 && ld <= 128 * ((kvp <= 128 ? 1 : kvp <= 256 ? 2 : kvp <= 512 ? 4 : 8) + 2) && stages_for(ld) >= 2; }
 size_t pm_latent_part_floats(int n_tokens, int H, int kvp) { return ((size_t) 512 + 2 * (size_t) n_tokens * ((H + 15) / 16)) * 16 * (kvp + 2); }
-int pm_launch_latent_decode(const pm_latent_layer & a, const pm_batch_dev & b, int n, int fused, int max_keys, hipStream_t st) {
+int pm_launch_latent_decode(const pm_latent_layer & a, const pm_batch_dev & b, int n, int fused, int max_keys, pm_split_merge * merge, hipStream_t st) {
     if (a.type != PM_BF16 || !pm_latent_decode_ok(a.kvp, a.ld) || n < 1) return PM355_E_UNSUPPORTED;
     int splits = splits_for(n, a.H, max_keys);
-    if (!a.part || !a.ticket || pm_latent_part_floats(n, a.H, a.kvp) > a.part_floats) splits = 1;
-    const int stages = stages_for(a.ld);
+    if (!a.part || pm_latent_part_floats(n, a.H, a.kvp) > a.part_floats) splits = 1;
+    const int stages = stages_for(a.ld), HT = (a.H + 15) / 16;
+    float * ml = a.part + (size_t) n * HT * splits * 16 * a.kvp;
     const size_t lds = (size_t) stages * a.ld * 2 * STEP + SCORES;
-    auto go = [&](auto kern) { pm_allow_big_lds((const void *) kern, lds); hipLaunchKernelGGL(kern, dim3(n, (a.H + 15) / 16, splits), dim3(DW * 64), lds, st, a, b, fused, splits, stages); return 0; };
-    return a.kvp <= 128 ? go(latent_decode_kernel<1>) : a.kvp <= 256 ? go(latent_decode_kernel<2>) : a.kvp <= 512 ? go(latent_decode_kernel<4>) : go(latent_decode_kernel<8>);
+    auto go = [&](auto kern) { pm_allow_big_lds((const void *) kern, lds); hipLaunchKernelGGL(kern, dim3(n, HT, splits), dim3(DW * 64), lds, st, a, b, fused, splits, stages, ml); };
+    if (a.kvp <= 128) go(latent_decode_kernel<1>); else if (a.kvp <= 256) go(latent_decode_kernel<2>); else if (a.kvp <= 512) go(latent_decode_kernel<4>); else go(latent_decode_kernel<8>);
+    if (merge) *merge = pm_split_merge{a.part, ml, splits, a.H};
+    else if (splits > 1) hipLaunchKernelGGL(latent_merge_kernel, dim3(n, a.H), dim3(256), 0, st, a, ml, splits);
+    return 0;
 }

@@ -27,17 +27,16 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
     const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 31, h_ = lane >> 5;
     const int wm = wave / (BN / WN), wn = wave % (BN / WN);
     // tile order: XCD x = blockIdx % 8 takes a contiguous run of tiles; runs walk blocks of 8 token tiles column by column
-    const int total = p.nt * p.nn, per = (total + 7) / 8;
+    const int nt = KIND == EXPERTS ? __builtin_amdgcn_readfirstlane(ld_g(p.tiles)) : p.nt;      // (the grid has room for the most tiles there can be)
+    const int total = nt * p.nn, per = (total + 7) / 8;
     const int slot = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if (slot >= total || (int) (blockIdx.x >> 3) >= per) return;
-    const int band = slot / (8 * p.nn), left = p.nt - band * 8, bh = left < 8 ? left : 8, in = slot - band * 8 * p.nn;
+    const int band = slot / (8 * p.nn), left = nt - band * 8, bh = left < 8 ? left : 8, in = slot - band * 8 * p.nn;
     int t0 = (band * 8 + in % bh) * BM, n_tok = p.T;
     const int n0 = (in / bh) * BN;
     const uint16_t * W = p.W;
     if constexpr (KIND == EXPERTS) {                       // t0, n_tok: sorted pairs of this tile
-        const int tile = band * 8 + in % bh;
-        if (tile >= __builtin_amdgcn_readfirstlane(ld_g(p.tiles))) return;
-        const int32_t * tt = p.tiles + 1 + 3 * tile;
+        const int32_t * tt = p.tiles + 1 + 3 * (band * 8 + in % bh);
         W += (int64_t) __builtin_amdgcn_readfirstlane(ld_g(tt)) * p.e_stride;
         t0 = __builtin_amdgcn_readfirstlane(ld_g(tt + 1)); n_tok = t0 + __builtin_amdgcn_readfirstlane(ld_g(tt + 2));
     }
@@ -102,6 +101,17 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
                 for (int n = 0; n < NI; ++n) acc[m][n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[m], b[n], acc[m][n], 0, 0, 0);
         }
     }
+    int * s_pair = (int *) smem;
+    float * s_weight = (float *) (smem + BM * 4);
+    if constexpr (KIND == EXPERTS) {                       // what the stores need about their rows
+        __syncthreads();
+        for (int i = threadIdx.x; i < BM; i += WAVES * 64) {
+            const int pair = ld_g(p.order + (t0 + i < n_tok ? t0 + i : n_tok - 1));
+            s_pair[i] = p.scatter ? pair : t0 + i;
+            s_weight[i] = p.weight ? ld_g(p.weight + pair) : 1.0f;
+        }
+        __syncthreads();
+    }
     // tokens are the tile's rows, W rows its columns: a register's 32 lanes store 32 consecutive outputs of one token
 #pragma unroll
     for (int n = 0; n < NI; ++n) {
@@ -136,13 +146,7 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
                 int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
                 float v = act_apply(p.act_fn, acc[m][n][e] + bias);
                 if (!ok || tok >= n_tok) continue;
-                if constexpr (KIND == EXPERTS) {
-                    if (p.weight || p.scatter) {
-                        const int pair = ld_g(p.order + tok);
-                        if (p.weight) v *= ld_g(p.weight + pair);
-                        if (p.scatter) tok = pair;
-                    }
-                }
+                if constexpr (KIND == EXPERTS) { v *= s_weight[tok - t0]; tok = s_pair[tok - t0]; }
                 st_type(p.y, (size_t) tok * p.ldy + col, p.y_type, v);
             }
     }
@@ -175,7 +179,9 @@ int pm_launch_dense_gemm(const pm_dense_args & a, hipStream_t st) {
 }
 
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st) {
-    return a.pro || a.group || a.type != PM_BF16 || a.T <= 64 ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
+    // (few rows of W: the prompt kernel's grid would leave most of the chip idle)
+    const bool narrow = a.n_store <= 256 && (long) ((a.T + 127) / 128) * ((a.n_store + 127) / 128) < 64;
+    return a.pro || a.group || a.type != PM_BF16 || a.T <= 64 || narrow ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
 }
 
 int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st) {

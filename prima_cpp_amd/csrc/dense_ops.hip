@@ -35,14 +35,38 @@ __device__ __forceinline__ float block_sum(float v, float * red) {
     return s;
 }
 
-// one token per workgroup; the first workgroups bring page tables, previous tokens and counters up to date (their readers are later launches; a portion's previous token
-// is read and replaced by the workgroup of its first token)
-__global__ __launch_bounds__(256) void embed_kernel(pm_embed_args a, pm_batch_dev b) {
-    __shared__ float red[4];
+// eight consecutive values from a 16-byte aligned row
+__device__ __forceinline__ void ld8(const void * p, size_t i, int type, float * v) {
+    if (type == PM_BF16) {
+        const u32x4 r = *(const PM_G u32x4 *) ((const uint16_t *) p + i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = bf2f((uint16_t) (r[e >> 1] >> (e & 1) * 16));
+    } else {
+        const f32x4 a = *(const PM_G f32x4 *) ((const float *) p + i), b = *(const PM_G f32x4 *) ((const float *) p + i + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { v[e] = a[e]; v[4 + e] = b[e]; }
+    }
+}
+__device__ __forceinline__ void st8(void * p, size_t i, int type, const float * v) {
+    if (type == PM_BF16) {
+        u32x4 r;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r[e] = (uint32_t) f2bf(v[2 * e]) | (uint32_t) f2bf(v[2 * e + 1]) << 16;
+        *(PM_G u32x4 *) ((uint16_t *) p + i) = r;
+    } else {
+        *(PM_G f32x4 *) ((float *) p + i) = f32x4{v[0], v[1], v[2], v[3]};
+        *(PM_G f32x4 *) ((float *) p + i + 4) = f32x4{v[4], v[5], v[6], v[7]};
+    }
+}
+// one token per workgroup, the row in registers (8 x EMBED_ROUNDS values per thread); the first workgroups bring page tables, previous tokens and counters up to date (their
+// readers are later launches; a portion's previous token is read and replaced by the workgroup of its first token)
+constexpr int EMBED_ROUNDS = 4;
+__global__ __launch_bounds__(1024) void embed_kernel(pm_embed_args a, pm_batch_dev b) {
+    __shared__ float red[16];
     const int t = blockIdx.x;
     if (t == 0) {
-        for (int i = threadIdx.x; i < b.n_upd[0]; i += 256) b.table[b.upd[2 * i]] = b.upd[2 * i + 1];
-        for (int i = threadIdx.x; i < a.n_clear; i += 256) a.clear[i] = 0;
+        for (int i = threadIdx.x; i < b.n_upd[0]; i += blockDim.x) b.table[b.upd[2 * i]] = b.upd[2 * i + 1];
+        for (int i = threadIdx.x; i < a.n_clear; i += blockDim.x) a.clear[i] = 0;
     }
     auto token = [&](int r) { const int k = b.tok[r]; return k < 0 ? b.last[b.seq[r]] : k; };
     const int tok = token(t);
@@ -53,17 +77,36 @@ __global__ __launch_bounds__(256) void embed_kernel(pm_embed_args a, pm_batch_de
         __syncthreads();                                   // (every wave has read prev)
         if (i == 0 && threadIdx.x == 0) b.prev[b.seq[t]] = token(t + b.left[t]);
     }
-    float s = 0.0f;
-    for (int c = threadIdx.x; c < a.Kp; c += 256) {
-        float v = c < a.width ? ld_any(a.embed, (size_t) tok * a.Kp + c, a.type) : 0.0f;
-        if (row >= 0 && c < a.width) v += ld_any(a.bigram, (size_t) row * a.Kp + c, a.type);
-        a.x[(size_t) t * a.Kp + c] = v;
-        s = fmaf(v, v, s);
-        if (a.out && !a.w2) st_type(a.out, (size_t) t * a.Kp + c, a.type, v);
+    float v[EMBED_ROUNDS][8], s = 0.0f;
+#pragma unroll
+    for (int i = 0; i < EMBED_ROUNDS; ++i) {
+        const int c = (i * (int) blockDim.x + (int) threadIdx.x) * 8;
+        if (c >= a.Kp) continue;
+        ld8(a.embed, (size_t) tok * a.Kp + c, a.type, v[i]);
+        if (row >= 0) {
+            float g[8];
+            ld8(a.bigram, (size_t) row * a.Kp + c, a.type, g);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[i][e] += g[e];
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s = fmaf(v[i][e], v[i][e], s);                       // (padding columns are zero)
     }
-    if (!a.out || !a.w2) return;
-    const float rs = 1.0f / sqrtf(block_sum(s, red) / (float) a.width + a.eps);
-    for (int c = threadIdx.x; c < a.Kp; c += 256) st_type(a.out, (size_t) t * a.Kp + c, a.type, c < a.width ? a.x[(size_t) t * a.Kp + c] * (rs * a.w2[c]) : 0.0f);
+    const float rs = a.out && a.w2 ? 1.0f / sqrtf(block_sum(s, red) / (float) a.width + a.eps) : 1.0f;
+#pragma unroll
+    for (int i = 0; i < EMBED_ROUNDS; ++i) {
+        const int c = (i * (int) blockDim.x + (int) threadIdx.x) * 8;
+        if (c >= a.Kp) continue;
+        st8(a.x, (size_t) t * a.Kp + c, PM_F32, v[i]);
+        if (!a.out) continue;
+        if (a.w2) {
+            float w[8];
+            ld8(a.w2, c, PM_F32, w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[i][e] *= rs * w[e];
+        }
+        st8(a.out, (size_t) t * a.Kp + c, a.type, v[i]);
+    }
 }
 __global__ void rope_table_kernel(const int32_t * pos, float base, int dims, float * cs) {
     const int half = dims / 2;
@@ -129,6 +172,67 @@ template <bool RES, int NTH, int VP> __global__ __launch_bounds__(NTH) void norm
     } else for (int c = threadIdx.x; c < width; c += NTH) st_type(out, (size_t) r * ldo + c, type, row[c] * (r2 * (RES && q.w2 ? q.w2[c] : 1.0f)));
 }
 
+// x[row] += norm(y[row]), out = the sum or its RMS norm with weight w2, four consecutive columns per thread and round: rows that are padded to multiples of 4
+template <int NTH, int VP> __global__ __launch_bounds__(NTH) void norm4_kernel(int type, pm_norm_args q, float * x, const void * y, int ldx, int ldy, void * out, int ldo) {
+    __shared__ float red[NTH / 64];
+    const int r = blockIdx.x, width = q.width;
+    float * xr = x + (size_t) r * ldx;
+    const int parts = q.parts ? q.parts : 1;
+    f32x4 v[VP], xv[VP];
+    float s = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+        const int c = (i * NTH + threadIdx.x) * 4;
+        v[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+        xv[i] = v[i];
+        if (c >= width) continue;
+        xv[i] = *(const PM_G f32x4 *) (xr + c);
+        for (int k = 0; k < parts; ++k) {
+            const size_t at = ((size_t) r * parts + k) * ldy + c;
+            if (q.y_type == PM_F32) v[i] += *(const PM_G f32x4 *) ((const float *) y + at);
+            else {
+                const u32x2 b = *(const PM_G u32x2 *) ((const uint16_t *) y + at);
+                v[i] += f32x4{bf2f((uint16_t) b[0]), bf2f((uint16_t) (b[0] >> 16)), bf2f((uint16_t) b[1]), bf2f((uint16_t) (b[1] >> 16))};
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { if (c + e >= width) v[i][e] = 0.0f; s += v[i][e]; }
+    }
+    const float mean = q.rms ? 0.0f : block_sum(s, red) / (float) width;
+    float s2 = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VP; ++i)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { const float d = (i * NTH + (int) threadIdx.x) * 4 + e < width ? v[i][e] - mean : 0.0f; s2 = fmaf(d, d, s2); }
+    const float rs = 1.0f / sqrtf(block_sum(s2, red) / (float) width + q.eps);
+    float s3 = 0.0f;
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+        const int c = (i * NTH + threadIdx.x) * 4;
+        if (c >= width) continue;
+        const f32x4 w = *(const PM_G f32x4 *) (q.w + c);
+        f32x4 bias = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (q.b) bias = *(const PM_G f32x4 *) (q.b + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { const float o = xv[i][e] + ((v[i][e] - mean) * rs * w[e] + bias[e]); v[i][e] = c + e < width ? o : 0.0f; s3 = fmaf(v[i][e], v[i][e], s3); }
+        *(PM_G f32x4 *) (xr + c) = v[i];
+    }
+    const float r2 = q.w2 ? 1.0f / sqrtf(block_sum(s3, red) / (float) width + q.eps) : 1.0f;
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+        const int c = (i * NTH + threadIdx.x) * 4;
+        if (c >= width) continue;
+        f32x4 o = v[i];
+        if (q.w2) {
+            const f32x4 w2 = *(const PM_G f32x4 *) (q.w2 + c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] *= r2 * w2[e];
+        }
+        if (type == PM_F32) *(PM_G f32x4 *) ((float *) out + (size_t) r * ldo + c) = o;
+        else *(PM_G u32x2 *) ((uint16_t *) out + (size_t) r * ldo + c) = u32x2{(uint32_t) f2bf(o[0]) | (uint32_t) f2bf(o[1]) << 16, (uint32_t) f2bf(o[2]) | (uint32_t) f2bf(o[3]) << 16};
+    }
+}
+
 // index of the first maximum of every row (src/llama-sampling.cpp:390-397), also kept per sequence for the next step
 __global__ __launch_bounds__(1024) void argmax_rows_kernel(const float * x, int n, int32_t * out, const int32_t * seq_of_row, int32_t * last) {
     __shared__ float bv[16]; __shared__ int bi[16];
@@ -163,7 +267,12 @@ void pm_launch_dense_fill(int type, void * dst, int K, int64_t N, int Kp, uint64
     const long n = (long) N * K, g = (n + 255) / 256;
     hipLaunchKernelGGL(fill_kernel, dim3((unsigned) (g < 65536 ? g : 65536)), dim3(256), 0, st, type, dst, K, n, Kp, seed, mean, amp);
 }
-void pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st) { hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, st, a, b); }
+int pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st) {
+    const int threads = a.Kp / 8 >= 1024 ? 1024 : (a.Kp / 8 + 63) / 64 * 64;
+    if (a.Kp % 64 || a.Kp > threads * 8 * EMBED_ROUNDS) return PM355_E_SHAPE;
+    hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(threads), 0, st, a, b);
+    return 0;
+}
 void pm_launch_rope_table(const int32_t * pos, int T, float base, int dims, float * cs, hipStream_t st) {
     hipLaunchKernelGGL(rope_table_kernel, dim3(T), dim3(64), 0, st, pos, base, dims, cs);
 }
@@ -180,6 +289,14 @@ template <bool RES> static void launch_norm(int type, const pm_norm_args & q, fl
     else go(norm_kernel<RES, 1024, 0>, 1024, (size_t) q.width * 4);
 }
 void pm_launch_add_norm(int type, const pm_norm_args & q, float * x, const void * y, int ldx, int ldy, int n_rows, void * out, int ldo, hipStream_t st) {
+    if (q.padded && out && n_rows > 16 && q.width <= 8192 && ldx % 4 == 0 && ldy % 4 == 0 && ldo % 4 == 0) {
+        auto go = [&](auto kern, int threads) { hipLaunchKernelGGL(kern, dim3(n_rows), dim3(threads), 0, st, type, q, x, y, ldx, ldy, out, ldo); };
+        if (q.width <= 1024) go(norm4_kernel<256, 1>, 256);
+        else if (q.width <= 2048) go(norm4_kernel<256, 2>, 256);
+        else if (q.width <= 4096) go(norm4_kernel<256, 4>, 256);
+        else go(norm4_kernel<512, 4>, 512);
+        return;
+    }
     launch_norm<true>(type, q, x, y, ldx, ldy, nullptr, n_rows, out, ldo, st);
 }
 void pm_launch_norm_rows(int type, const pm_norm_args & q, const float * x, int ldx, const int32_t * rows, int n_rows, void * out, int ldo, hipStream_t st) {

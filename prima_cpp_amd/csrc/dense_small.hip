@@ -16,7 +16,7 @@ enum { DENSE = 0, PAIR = 1, CONCAT = 2, SORTED = 3 };
 struct SmallP {
     const void * W; const void * act; void * y; const float * bias; pm_add_norm pro;
     int K, T, lda, ldy, y_type, n_store, act_fn;
-    int group, g_act, g_out, g_store;
+    int group, g_act, g_out, g_store; pm_split_merge merge;
     // experts: values between two of them; SORTED: rows in / out are sorted pairs (in_sorted / out_sorted) or tokens / pairs
     pm_route r; int64_t e_stride; int in_sorted, out_sorted, weigh;
 };
@@ -188,7 +188,35 @@ template <typename T, int NT, int RM, int SRC, int EXP> __global__ __launch_boun
         T * rows = (T *) (smem + 8 * NT * RM * 1024);
         const int here = n_tok - t0 < TOK ? n_tok - t0 : TOK;
         if (SRC > 0) norm.finish(p, rows, ldl, red, wave, lane);
-        else {
+        else if (EXP == DENSE && sizeof(T) == 2 && p.merge.part) {
+            // the activations are sums over key splits (wave t: the shares of token t's splits)
+            __shared__ float share[8 * 64];
+            const int h = r0 / p.group < p.merge.H ? r0 / p.group : p.merge.H - 1;
+            const size_t ht = (p.merge.H + 15) / 16;
+            const pm_split_merge & q = p.merge;
+            if (wave < here) {
+                const size_t slot = (size_t) (t0 + wave) * ht + h / 16;
+                const float * ml = q.ml + ((slot * q.splits + (lane < q.splits ? lane : 0)) * 16 + h % 16) * 2;
+                const float m = lane < q.splits ? ld_g(ml) : -1e30f, l = lane < q.splits ? ld_g(ml + 1) : 0.0f, f = __builtin_amdgcn_exp2f(m - wave_max(m));
+                share[wave * 64 + lane] = f / wave_sum(l * f);
+            }
+            __syncthreads();
+            const int n2 = kk / 2;
+            for (int i = threadIdx.x; i < here * n2; i += 512) {
+                const int t = i / n2, c = (i - t * n2) * 2;
+                const float * src = q.part + ((((size_t) (t0 + t) * ht + h / 16) * q.splits) * 16 + h % 16) * kk + c;
+                float a0 = 0.0f, a1 = 0.0f;
+                for (int s0 = 0; s0 < q.splits; s0 += 16) {
+                    float2 v[16];
+#pragma unroll
+                    for (int s = 0; s < 16; ++s) v[s] = __builtin_bit_cast(float2, *(const PM_G u32x2 *) (src + (size_t) (s0 + s < q.splits ? s0 + s : 0) * 16 * kk));
+#pragma unroll
+                    for (int s = 0; s < 16; ++s) { const float w = s0 + s < q.splits ? share[t * 64 + s0 + s] : 0.0f; a0 = fmaf(v[s].x, w, a0); a1 = fmaf(v[s].y, w, a1); }
+                }
+                rows[t * ldl + c] = from_f<T>(a0); rows[t * ldl + c + 1] = from_f<T>(a1);
+            }
+            __syncthreads();
+        } else {
             const int n16 = kk / EPL;
             for (int t = 0; t < here; ++t) {
                 const T * src = row_in(t0 + t);
@@ -300,7 +328,8 @@ template <typename T> int launch_type(const pm_dense_args & a, const SmallP & p,
     }
     if constexpr (sizeof(T) == 2)
         if (a.T <= 8 && (size_t) a.T * (a.K * 2 + 16) <= LDS_ACT) return rm == 1 ? launch<T, 1, 1, -1>(p, N, 0, st) : launch<T, 1, 2, -1>(p, N, 0, st);
-    const bool wide = N / 32 >= 512;
+    const bool wide = N / 32 >= 512 || (sizeof(T) == 2 && a.T > 64 && (long) (N / 32) * ((a.T + 63) / 64) >= 128);
+    if (a.merge) return PM355_E_SHAPE;                     // (pm_dense_merge_ok)
     if (a.T <= 16) return wide ? launch<T, 1, 2, 0>(p, N, 0, st) : launch<T, 1, 1, 0>(p, N, 0, st);
     if (a.T <= 32) return wide ? launch<T, 2, 2, 0>(p, N, 0, st) : launch<T, 2, 1, 0>(p, N, 0, st);
     if constexpr (sizeof(T) == 2) if (wide) return launch<T, 4, 2, 0>(p, N, 0, st);
@@ -332,6 +361,7 @@ template <typename T> int experts_type(const pm_expert_args & a, hipStream_t st)
 
 } // namespace
 
+bool pm_dense_merge_ok(int T, int K) { return T <= 8 && (size_t) T * (K * 2 + 16) <= LDS_ACT; }
 bool pm_dense_pro_ok(int T, int width) { return T >= 1 && T <= 4 && width * (T == 1 ? 1 : T == 2 ? 2 : 4) <= PRO_MAX; }
 
 int pm_launch_dense_small(const pm_dense_args & a, hipStream_t st) {
@@ -339,6 +369,8 @@ int pm_launch_dense_small(const pm_dense_args & a, hipStream_t st) {
     p.W = a.W; p.act = a.act; p.y = a.y; p.bias = a.bias; p.K = a.K; p.T = a.T; p.lda = a.lda; p.ldy = a.ldy; p.y_type = a.y_type; p.n_store = a.n_store; p.act_fn = a.act_fn;
     p.group = a.group; p.g_act = a.g_act; p.g_out = a.g_out; p.g_store = a.g_store;
     if (a.pro) p.pro = *a.pro;
+    if (a.merge) p.merge = *a.merge;
+    if (a.merge && (!a.group || a.type != PM_BF16 || a.merge->splits < 1 || a.merge->splits > 64 || !pm_dense_merge_ok(a.T, a.K))) return PM355_E_SHAPE;
     if (a.K % 64 || a.N % 64 || (!a.group && a.n_store > a.N) || a.T < 1 || (a.type != PM_BF16 && a.type != PM_F32)) return PM355_E_SHAPE;
     if (a.group && (a.group % 32 || a.pro || a.bias || (size_t) a.g_act * pm_dense_bytes(a.type) % 16)) return PM355_E_SHAPE;
     return a.type == PM_BF16 ? launch_type<uint16_t>(a, p, st) : launch_type<float>(a, p, st);

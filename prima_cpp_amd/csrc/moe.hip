@@ -68,18 +68,25 @@ __global__ __launch_bounds__(1024) void route_one_kernel(pm_route r, int T, int 
     }
 }
 
-__global__ __launch_bounds__(256) void route_select_kernel(pm_route r, int T) {
+// 32 tokens per workgroup: places among its own pairs by LDS counters, then one global counter update per expert
+constexpr int SEL_TOK = 32;
+__global__ __launch_bounds__(1024) void route_select_kernel(pm_route r, int T) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
-    float * s = sm + wave * (r.E + r.groups + 2 * r.top), * gs = s + r.E, * w = gs + r.groups;
-    int * ids = (int *) (w + r.top);
-    if (t >= T) return;
-    route_token(r.logits + (size_t) t * r.ldl, r.E, r.top, r.groups, r.keep, s, gs, ids, w);
-    for (int k = lane; k < r.top; k += 64) {
-        const int p = t * r.top + k;
-        r.id[p] = ids[k]; r.w[p] = w[k];
-        r.pos[p] = atomicAdd(r.count + ids[k], 1);
+    const int wave = threadIdx.x >> 6, t0 = blockIdx.x * SEL_TOK, n = (T - t0 < SEL_TOK ? T - t0 : SEL_TOK) * r.top;
+    int * count = (int *) sm, * ids = count + r.E;
+    float * w = (float *) (ids + SEL_TOK * r.top), * s = w + SEL_TOK * r.top + wave * (r.E + r.groups);
+    for (int e = threadIdx.x; e < r.E; e += 1024) count[e] = 0;
+    for (int i = wave; i < SEL_TOK && t0 + i < T; i += 16)
+        route_token(r.logits + (size_t) (t0 + i) * r.ldl, r.E, r.top, r.groups, r.keep, s, s + r.E, ids + i * r.top, w + i * r.top);
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += 1024) {
+        r.id[t0 * r.top + i] = ids[i]; r.w[t0 * r.top + i] = w[i];
+        ((int *) w)[i] = atomicAdd(count + ids[i], 1);     // (the weight has been stored: its place takes over)
     }
+    __syncthreads();
+    for (int e = threadIdx.x; e < r.E; e += 1024) if (count[e]) count[e] = atomicAdd(r.count + e, count[e]);
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += 1024) r.pos[t0 * r.top + i] = count[ids[i]] + ((int *) w)[i];
 }
 __global__ __launch_bounds__(256) void route_place_kernel(pm_route r, int pairs, int want_tiles) {
     extern __shared__ __attribute__((aligned(16))) int cnt[];
@@ -105,8 +112,8 @@ void pm_launch_route(const pm_route & r, int T, int want_tiles, hipStream_t st) 
         pm_allow_big_lds((const void *) route_one_kernel, lds);
         if (lds <= 150 * 1024) { hipLaunchKernelGGL(route_one_kernel, dim3(1), dim3(1024), lds, st, r, T, want_tiles); return; }
     }
-    const size_t lds = (size_t) 4 * (r.E + r.groups + 2 * r.top) * 4;
+    const size_t lds = ((size_t) r.E + 2 * SEL_TOK * r.top + 16 * (r.E + r.groups)) * 4;      // (at most 150 KB: E, groups <= 1024, top <= 64)
     pm_allow_big_lds((const void *) route_select_kernel, lds);
-    hipLaunchKernelGGL(route_select_kernel, dim3((T + 3) / 4), dim3(256), lds, st, r, T);
+    hipLaunchKernelGGL(route_select_kernel, dim3((T + SEL_TOK - 1) / SEL_TOK), dim3(1024), lds, st, r, T);
     hipLaunchKernelGGL(route_place_kernel, dim3((pairs + 255) / 256), dim3(256), (size_t) (2 * r.E + 1) * 4, st, r, pairs, want_tiles);
 }

@@ -20,6 +20,8 @@ struct pm_add_norm {
     float * x_out; int ldo;
     int rms; const float * w2; void * act_out; int ld_act;
 };
+// attention outputs of one head per group that are still split by keys: part [T x head tiles][splits][16 heads][K] sums, ml [..][splits][16][maximum (log2 units), sum]
+struct pm_split_merge { const float * part, * ml; int splits, H; };
 struct pm_dense_args {
     int type; const void * W; int K, N;                 // N: rows of W that exist (multiple of 64)
     const void * act; int lda; int T;
@@ -29,8 +31,10 @@ struct pm_dense_args {
     // group != 0 (a multiple of 32; the small-batch kernel, any T): one matrix per group of `group` rows (attention heads): group g multiplies the K activations from column
     // g * g_act on, its first g_store rows go to the columns from g * g_out on
     int group, g_act, g_out, g_store;
+    const pm_split_merge * merge;                       // != null (pm_dense_merge_ok, bf16, group = a head): the activations are merged from key splits on the way in
 };
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st);                    // picks the small-batch or the prompt kernel
+bool pm_dense_merge_ok(int T, int K);
 bool pm_dense_pro_ok(int T, int width);
 
 // f32 / bf16 host-order matrix [N][K] -> [rows at dst_row][Kp] of `type` (columns >= K stay as they are: zero from allocation). group > 0: rows come in groups of `group`,
@@ -59,9 +63,10 @@ struct pm_embed_args {
     const float * w2; float eps; int32_t * clear; int n_clear;
     float * x; void * out;
 };
-void pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st);
+int  pm_launch_stack_embed(const pm_embed_args & a, const pm_batch_dev & b, int T, hipStream_t st);
 // x += norm(y); out = x (or, with w2, x / rms(x) * w2) in T. parts > 0: y is the sum of `parts` rows, y[row * parts ..]; y_type: of y
-struct pm_norm_args { int rms; const float * w, * b, * w2; float eps; int width; int y_type, parts; };
+// padded: rows (and w, b, w2) may be read and x and out written up to the next multiple of 4 columns
+struct pm_norm_args { int rms; const float * w, * b, * w2; float eps; int width; int y_type, parts; bool padded; };
 void pm_launch_add_norm(int type, const pm_norm_args & n, float * x, const void * y, int ldx, int ldy, int n_rows, void * out, int ldo, hipStream_t st);
 // out[r] = norm(x[rows[r]]) in T (rows: gather list or null)
 void pm_launch_norm_rows(int type, const pm_norm_args & n, const float * x, int ldx, const int32_t * rows, int n_rows, void * out, int ldo, hipStream_t st);
@@ -106,14 +111,15 @@ struct pm_latent_layer {
     void * qa;                              // [T][H][ld] queries in the latent | rotated part
     void * out; int ldo;                    // [T][ldo]: H x kvp weighted latents
     const float * cs;                       // [T][rot_dims / 2][cos, sin]
-    float * part; unsigned * ticket; size_t part_floats;
+    float * part; size_t part_floats;
 };
 // query latents normed (cq != null), latents normed and keys rotated into the cache (kv_norm != null)
 void pm_launch_latent_prepare(const pm_latent_layer & a, const pm_batch_dev & b, int T, hipStream_t st);
 // rotates the queries' rotated part: in place in qh, and into qa
 void pm_launch_latent_rotate(const pm_latent_layer & a, int T, hipStream_t st);
-// tokens 0 .. n - 1 of the step. fused: the cache store and the rotation of the queries happen inside (every entry is one token)
-int  pm_launch_latent_decode(const pm_latent_layer & a, const pm_batch_dev & b, int n, int fused, int max_keys, hipStream_t st);
+// tokens 0 .. n - 1 of the step. fused: the cache store and the rotation of the queries happen inside (every entry is one token). Keys may be split over workgroups: with
+// merge != null the sums stay split for the value product (merge->splits > 1), otherwise `out` is complete
+int  pm_launch_latent_decode(const pm_latent_layer & a, const pm_batch_dev & b, int n, int fused, int max_keys, pm_split_merge * merge, hipStream_t st);
 void pm_launch_latent_plain(const pm_latent_layer & a, const pm_batch_dev & b, int n, hipStream_t st);
 bool pm_latent_decode_ok(int kvp, int ld);
 size_t pm_latent_part_floats(int n_tokens, int H, int kvp);
@@ -202,7 +208,13 @@ __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + __ex
 // first key position the query at `pos` sees
 __device__ __forceinline__ int first_key(int pos, int mask, int size) { return mask == 1 ? pos - pos % size : mask == 2 && pos >= size ? pos - size + 1 : 0; }
 __device__ __forceinline__ float silu32(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// log(1 + e^z) = max(z, 0) + log(1 + u), u = e^-|z|; log(1 + u) = 2 atanh(s), s = u / (2 + u) <= 1/3, by the series of atanh (next term: 1e-9 of the sum)
+__device__ __forceinline__ float softplus_f(float z) {
+    const float u = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z)), s = u * __builtin_amdgcn_rcpf(2.0f + u), q = s * s;
+    float p = 1.0f / 17;
+    p = fmaf(p, q, 1.0f / 15); p = fmaf(p, q, 1.0f / 13); p = fmaf(p, q, 1.0f / 11); p = fmaf(p, q, 1.0f / 9); p = fmaf(p, q, 1.0f / 7); p = fmaf(p, q, 0.2f); p = fmaf(p, q, 1.0f / 3);
+    return fmaxf(z, 0.0f) + 2.0f * fmaf(s * q, p, s);
+}
 // activation functions of the dense products (PM355_ACT_*)
 __device__ __forceinline__ float act_apply(int fn, float v) {
     if (fn == 1) { v = fmaxf(v, 0.0f); v *= v; }

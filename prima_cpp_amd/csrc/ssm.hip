@@ -65,8 +65,17 @@ template <int NG> struct States { f32x4 s[NG], a[NG]; };
 __device__ __forceinline__ f32x4 decay4(f32x4 a, float dt) {
     return f32x4{__builtin_amdgcn_exp2f(a[0] * dt), __builtin_amdgcn_exp2f(a[1] * dt), __builtin_amdgcn_exp2f(a[2] * dt), __builtin_amdgcn_exp2f(a[3] * dt)};
 }
+// sum over groups of n lanes (a power of two, the same in every lane): data-parallel moves inside a row of 16 lanes
+template <int CTRL> __device__ __forceinline__ float moved(float v) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
+}
 __device__ __forceinline__ float lanes_sum(float v, int n) {
-    for (int o = 1; o < n; o *= 2) v += __shfl_xor(v, o);
+    if (n > 1) v += moved<0xB1>(v);                        // quad_perm 1 0 3 2
+    if (n > 2) v += moved<0x4E>(v);                        // quad_perm 2 3 0 1
+    if (n > 4) v += moved<0x141>(v);                       // row_half_mirror: the other quad
+    if (n > 8) v += moved<0x140>(v);                       // row_mirror: the other half row
+    if (n > 16) v += __shfl_xor(v, 16);
+    if (n > 32) v += __shfl_xor(v, 32);
     return v;
 }
 
@@ -121,7 +130,8 @@ template <typename T, int NG, int PHASE> __global__ __launch_bounds__(256) void 
     const bool last = ch.j == ch.n_chunks - 1;
     if (PHASE == 0 && last) return;
     const int cpb = 256 / lpc, sub = threadIdx.x % lpc, cl = threadIdx.x / lpc, c0 = blockIdx.y * cpb, c = c0 + cl, cc = c < a.inner ? c : a.inner - 1;
-    float * s_dt = sm, * s_dx = s_dt + TT * cpb, * s_y = s_dx + TT * cpb, * s_B = s_y + TT * cpb, * s_C = s_B + TT * a.sp;
+    float2 * s_dd = (float2 *) sm;                         // (step size, step size * input)
+    float * s_y = (float *) (s_dd + TT * cpb), * s_B = s_y + TT * cpb, * s_C = s_B + TT * a.sp;
     States<NG> st;
     const size_t at = (size_t) cc * a.sp + sub * 4;
     float * E = a.E + (size_t) (ch.e_base + ch.j) * a.inner * a.sp + at, * S = a.S + (size_t) ch.seq * a.inner * a.sp + at;
@@ -138,29 +148,31 @@ template <typename T, int NG, int PHASE> __global__ __launch_bounds__(256) void 
     for (int t0 = 0; t0 < ch.n; t0 += TT) {
         const int nt = ch.n - t0 < TT ? ch.n - t0 : TT;
         __syncthreads();
-        for (int i = threadIdx.x; i < nt * cpb; i += 256) {
+        for (int i = threadIdx.x; i < TT * cpb; i += 256) {       // (tokens past the end: steps of size 0 change nothing)
             const int t = i / cpb, k = c0 + i % cpb;
             const size_t r = (size_t) (ch.row + t0 + t);
             float dt = 0.0f, x = 0.0f;
-            if (k < a.inner) { dt = softplus_f(a.dt[r * a.innerp + k]); x = to_f<T>(((const T *) a.xc)[r * a.innerp + k]); }
-            s_dt[i] = dt; s_dx[i] = dt * x;
+            if (k < a.inner && t < nt) { dt = softplus_f(a.dt[r * a.innerp + k]); x = to_f<T>(((const T *) a.xc)[r * a.innerp + k]); }
+            s_dd[i] = make_float2(dt, dt * x);
         }
-        for (int i = threadIdx.x; i < nt * a.sp; i += 256) {
+        for (int i = threadIdx.x; i < TT * a.sp; i += 256) {
             const int t = i / a.sp, n = i % a.sp;
             const T * f = (const T *) a.f + (size_t) (ch.row + t0 + t) * a.ldf + a.dtp;
-            s_B[i] = n < a.state ? to_f<T>(f[n]) : 0.0f;
-            if (PHASE == 1) s_C[i] = n < a.state ? to_f<T>(f[a.state + n]) : 0.0f;
+            const bool on = n < a.state && t < nt;
+            s_B[i] = on ? to_f<T>(f[n]) : 0.0f;
+            if (PHASE == 1) s_C[i] = on ? to_f<T>(f[a.state + n]) : 0.0f;
         }
         __syncthreads();
-        for (int t = 0; t < nt; ++t) {
-            const float dt = s_dt[t * cpb + cl], dx = s_dx[t * cpb + cl];
-            if (PHASE == 0) sum += dt;
+#pragma unroll 4
+        for (int t = 0; t < TT; ++t) {
+            const float2 dd = s_dd[t * cpb + cl];
+            if (PHASE == 0) sum += dd.x;
             float y = 0.0f;
 #pragma unroll
             for (int g = 0; g < NG; ++g) {
-                const f32x4 B = *(const f32x4 *) (s_B + t * a.sp + sub * 4 + g * lpc * 4), dec = decay4(st.a[g], dt);
+                const f32x4 B = *(const f32x4 *) (s_B + t * a.sp + sub * 4 + g * lpc * 4), dec = decay4(st.a[g], dd.x);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) st.s[g][e] = fmaf(dec[e], st.s[g][e], dx * B[e]);
+                for (int e = 0; e < 4; ++e) st.s[g][e] = fmaf(dec[e], st.s[g][e], dd.y * B[e]);
                 if (PHASE == 1) {
                     const f32x4 C = *(const f32x4 *) (s_C + t * a.sp + sub * 4 + g * lpc * 4);
 #pragma unroll

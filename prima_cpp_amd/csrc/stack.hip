@@ -450,7 +450,6 @@ int pm_stack::finalize_pool(int max_tokens_, int n_seq, int64_t pool_tokens) {
         const pm355_layer_spec & s = L.s;
         if (s.mixer == PM355_MIXER_ATTENTION) groups = std::max(groups, s.n_head_kv * ((s.n_head / s.n_head_kv + 15) / 16));
         if (s.mixer == PM355_MIXER_LATENT) {
-            groups = std::max(groups, (s.n_head + 15) / 16);
             n_cq = std::max(n_cq, (size_t) L.uq.Kp); n_qa = std::max(n_qa, (size_t) s.n_head * L.ld); n_ol = std::max(n_ol, (size_t) s.n_head * L.kvp);
             if (L.mask_list >= 0) { n_xk = std::max(n_xk, (size_t) s.n_head * PM_PAGE * L.dkp); n_xv = std::max(n_xv, (size_t) s.n_head * PM_PAGE * L.dvp); }
             bool known = false;
@@ -642,7 +641,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
     const int rms = d.norm == PM355_NORM_RMS;
     auto norm_b = [&](float * b) -> const float * { return rms ? nullptr : b; };
     auto settle = [&](const float * pre) {
-        if (pend.on) pm_launch_add_norm(ty, pm_norm_args{rms, pend.w, pend.b, pre, d.norm_eps, d.n_embd, pend.type, pend.parts}, x[cur], pend.parts ? yrows : (void *) y, Wp, Wp, T, xb, Wp, st);
+        if (pend.on) pm_launch_add_norm(ty, pm_norm_args{rms, pend.w, pend.b, pre, d.norm_eps, d.n_embd, pend.type, pend.parts, true}, x[cur], pend.parts ? yrows : (void *) y, Wp, Wp, T, xb, Wp, st);
         pend.on = false;
     };
     // W . (residual stream, normed by `pre` where the design norms in front of a sublayer); keep: the activations are read again from xb
@@ -695,8 +694,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
         pm_latent_layer a{};
         a.type = ty; a.H = s.n_head; a.dim = s.k_dim; a.rot = s.rot_dim; a.rot_dims = s.rot_dims; a.kv_rank = s.kv_rank; a.kvp = L.kvp; a.ld = L.ld; a.scale = s.scale; a.eps = d.norm_eps;
         a.mask = s.mask; a.mask_size = s.mask_size; a.cache = L.kc; a.raw = raw; a.ldraw = L.proj.Np; a.raw_type = raw_type; a.q_rank = s.q_rank; a.q_norm = L.dq_norm;
-        a.ld_cq = L.uq.Kp; a.kv_norm = s.kv_from < 0 ? L.dkv_norm : nullptr; a.qh = q; a.qs = L.qs; a.qa = qa; a.out = ol; a.ldo = s.n_head * L.kvp; a.part = part; a.ticket = ticket;
-        a.part_floats = part_floats;
+        a.ld_cq = L.uq.Kp; a.kv_norm = s.kv_from < 0 ? L.dkv_norm : nullptr; a.qh = q; a.qs = L.qs; a.qa = qa; a.out = ol; a.ldo = s.n_head * L.kvp; a.part = part; a.part_floats = part_floats;
         for (auto & r : ropes) if (r.first == std::make_pair(s.rot_base, s.rot_dims)) a.cs = r.second;
         void * out = att[s.n_head * s.v_dim];
         const int hq = s.n_head * L.qs;
@@ -724,9 +722,11 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
             g.group = L.kvp; g.g_act = L.qs; g.g_out = L.ld; g.g_store = L.kvp;
             rc = pm_launch_dense(g, st);
             if (rc) return rc;
-            if (mfma) rc = pm_launch_latent_decode(a, p.b, rows, inside, seen_keys(s), st);
+            pm_split_merge split{nullptr, nullptr, 1, 0};
+            if (mfma) rc = pm_launch_latent_decode(a, p.b, rows, inside, seen_keys(s), pm_dense_merge_ok(rows, L.uv.Kp) ? &split : nullptr, st);
             else pm_launch_latent_plain(a, p.b, rows, st);
             if (rc) return rc;
+            if (split.splits > 1) g.merge = &split;
             g.W = L.uv.d; g.K = L.uv.Kp; g.N = L.uv.Np; g.act = ol; g.lda = a.ldo; g.y = out; g.ldy = L.out.Kp; g.n_store = s.n_head * s.v_dim;
             g.group = L.vrows; g.g_act = L.kvp; g.g_out = s.v_dim; g.g_store = s.v_dim;
             rc = pm_launch_dense(g, st);
@@ -785,7 +785,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
     pm_embed_args em{};
     em.type = ty; em.embed = embed.d; em.Kp = Wp; em.width = d.n_embd; em.bigram = bigram.d; em.buckets = d.bigram_buckets; em.mul_prev = d.bigram_mul_prev; em.mul_cur = d.bigram_mul_cur;
     em.w2 = layers[0].pre1; em.eps = d.norm_eps; em.clear = counts; em.n_clear = T > PM_ROUTE_PAIR_MAX ? n_moe * max_E : 0; em.x = x[0]; em.out = xb;
-    pm_launch_stack_embed(em, p.b, T, st);
+    if (const int rc = pm_launch_stack_embed(em, p.b, T, st)) return fail(rc, "batch: embedding");
     for (auto & r : ropes) pm_launch_rope_table(p.b.pos, T, r.first.first, r.first.second, r.second, st);
     for (auto & L : layers) {
         const pm355_layer_spec & s = L.s;
