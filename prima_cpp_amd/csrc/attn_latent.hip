@@ -27,10 +27,41 @@ template <typename F> __device__ __forceinline__ float rotated(const F & at, int
     return at(i);
 }
 // the token's cache row from its projections: scale of the latent's norm (one wave), then n threads store it
+// (loops of predicated loads would wait for one load after the other: these ask for eight at a time, indexes clamped)
 __device__ __forceinline__ float latent_scale(const pm_latent_layer & a, int t) {
+    const size_t at = (size_t) t * a.ldraw + a.q_rank;
     float s = 0.0f;
-    for (int d = threadIdx.x & 63; d < a.kv_rank; d += 64) { const float v = ld_any(a.raw, (size_t) t * a.ldraw + a.q_rank + d, a.raw_type); s = fmaf(v, v, s); }
+    for (int d0 = threadIdx.x & 63; d0 < a.kv_rank; d0 += 512) {
+        float v[8];
+        if (a.raw_type == PM_F32) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] = ld_g((const float *) a.raw + at + (d0 + 64 * j < a.kv_rank ? d0 + 64 * j : d0));
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] = bf2f(ld_g((const uint16_t *) a.raw + at + (d0 + 64 * j < a.kv_rank ? d0 + 64 * j : d0)));
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) s = d0 + 64 * j < a.kv_rank ? fmaf(v[j], v[j], s) : s;
+    }
     return 1.0f / sqrtf(wave_sum(s) / (float) a.kv_rank + a.eps);
+}
+// entries r0 .. r0 + 7 of a rotated bf16 vector, zero from `rot` on
+__device__ __forceinline__ bf16x8 rotated8(const uint16_t * q, int r0, int rot, int rot_dims, const float * cs) {
+    const int half = rot_dims / 2;
+    float u[8], w[8], c[8], s[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const int r = r0 + e < rot ? r0 + e : rot - 1, i = r < half ? r : r < 2 * half ? r - half : 0, o = r < half ? r + half : r < 2 * half ? r - half : r;
+        u[e] = bf2f(ld_g(q + r)); w[e] = bf2f(ld_g(q + o)); c[e] = ld_g(cs + 2 * i); s[e] = ld_g(cs + 2 * i + 1);
+    }
+    bf16x8 y;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const int r = r0 + e;
+        const float t = r < half ? u[e] * c[e] - w[e] * s[e] : u[e] * c[e] + w[e] * s[e];
+        y[e] = (__bf16) (r >= rot ? 0.0f : r < 2 * half ? t : u[e]);
+    }
+    return y;
 }
 template <typename T> __device__ __forceinline__ void store_row(const pm_latent_layer & a, int t, T * row, float rs, int i0, int n) {
     const size_t at = (size_t) t * a.ldraw + a.q_rank;
@@ -185,10 +216,7 @@ template <int VT> __global__ __launch_bounds__(DW * 64) void latent_decode_kerne
         q[i] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
         if (kq + 4 * i >= ks) continue;
         if (k < a.kvp || !fused) q[i] = __builtin_bit_cast(bf16x8, *(const PM_G u32x4 *) (qa + k));
-        else for (int e = 0; e < 8; ++e) {
-            const int r = k - a.kvp + e;
-            if (r < a.rot) q[i][e] = (__bf16) rotated([&](int j) { return bf2f(qr[j]); }, r, a.rot_dims, a.cs + (size_t) t * a.rot_dims);
-        }
+        else q[i] = rotated8(qr, k - a.kvp, a.rot, a.rot_dims, a.cs + (size_t) t * a.rot_dims);
         if (lr >= nh) q[i] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
     }
     const uint32_t krow = 8 * (lr >> 2) + 4 * kt + (lr & 3);            // key of score row lr

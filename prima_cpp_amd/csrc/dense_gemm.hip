@@ -7,7 +7,7 @@
 #include "pm355_dense.h"
 #include "pm355_kernels.h"
 #include "../../include/prima_mi355.h"
-#include <stdlib.h>
+#include <type_traits>
 
 namespace {
 
@@ -21,7 +21,9 @@ struct GemmP {
     const int32_t * pages; int H, per, rows_h, pad;              // heads, values per head, rows of W per head, padded head size of the output
 };
 
-template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__(BM / WM * (BN / WN) * 64) void dense_gemm_kernel(GemmP p) {
+template <int N> __device__ __forceinline__ void vm_wait() { asm volatile("s_waitcnt vmcnt(%0)" :: "n"(N) : "memory"); }
+
+template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __launch_bounds__(BM / WM * (BN / WN) * 64) void dense_gemm_kernel(GemmP p) {
     constexpr int WAVES = BM / WM * (BN / WN), MI = WM / 32, NI = WN / 32, PIECES = (BM + BN) / 8 / WAVES, STAGE = (BM + BN) * 128;
     extern __shared__ __attribute__((aligned(1024))) char smem[];
     const int wave = __builtin_amdgcn_readfirstlane((int) threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 31, h_ = lane >> 5;
@@ -42,6 +44,7 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
     }
 
     // DMA pieces of this wave (8 rows of 128 bytes each): the first half of the waves brings the tokens, the second half the rows of W
+    static_assert(STAGES == 2 || STAGES == 4, "stages are found by a mask, waits are spelled for these");
     static_assert(BM == BN, "a wave's pieces belong to one operand");
     const bool tok = wave < WAVES / 2;
     const char * base = tok ? (const char *) (KIND == VALUES ? W + (size_t) t0 * p.K : p.X + (KIND == EXPERTS ? 0 : (size_t) t0 * p.lda)) : (const char *) (W + (size_t) n0 * p.K);
@@ -81,24 +84,38 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
 #pragma unroll
     for (int n = 0; n < NI; ++n) { const int r = BM + wn * WN + n * 32 + lr; brow[n] = (uint32_t) r * 128u; bsw[n] = (r >> 1) & 7; }
 
+    float bias[NI];
+#pragma unroll
+    for (int n = 0; n < NI; ++n) { const int col = n0 + wn * WN + n * 32 + lr; bias[n] = KIND == DENSE && p.bias && col < p.n_store ? ld_g(p.bias + col) : 0.0f; }
     const int steps = p.K >> 6;
-    request(0, 0);
+#pragma unroll
+    for (int i = 0; i < STAGES - 1; ++i) if (i < steps) request(i, i);
     for (int k = 0; k < steps; ++k) {
-        pm_vm_drain();                                     // this step's lines have landed ..
-        __syncthreads();                                   // .. for every wave, and every wave is done with the other stage
-        if (k + 1 < steps) request(k + 1, (k + 1) & 1);
-        const char * s = smem + (k & 1) * STAGE;
+        const int ahead = steps - 1 - k;                   // this step's lines have landed (requests complete in order) ..
+        if (STAGES > 2 && ahead >= STAGES - 2) vm_wait<PIECES * (STAGES - 2)>();
+        else if (STAGES > 3 && ahead == 1) vm_wait<PIECES>();
+        else vm_wait<0>();
+        __syncthreads();                                   // .. for every wave, and every wave is done with the stage in front of this one
+        if (k + STAGES - 1 < steps) request(k + STAGES - 1, (k + STAGES - 1) & (STAGES - 1));
+        const char * s = smem + (k & (STAGES - 1)) * STAGE;
+        // fragments of the next 16 k are on their way while this 16 k's products run
+        bf16x8 a[2][MI], b[2][NI];
+        auto read = [&](int j) __attribute__((always_inline)) {
+#pragma unroll
+            for (int n = 0; n < NI; ++n) b[j & 1][n] = *(const bf16x8 *) (s + brow[n] + (uint32_t) (((j * 2 + h_) ^ bsw[n]) * 16));
+#pragma unroll
+            for (int m = 0; m < MI; ++m) a[j & 1][m] = *(const bf16x8 *) (s + arow[m] + (uint32_t) (((j * 2 + h_) ^ asw[m]) * 16));
+        };
+        read(0);
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            bf16x8 a[MI], b[NI];
-#pragma unroll
-            for (int n = 0; n < NI; ++n) b[n] = *(const bf16x8 *) (s + brow[n] + (uint32_t) (((j * 2 + h_) ^ bsw[n]) * 16));
-#pragma unroll
-            for (int m = 0; m < MI; ++m) a[m] = *(const bf16x8 *) (s + arow[m] + (uint32_t) (((j * 2 + h_) ^ asw[m]) * 16));
+            if (j < 3) read(j + 1);
+            __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
             for (int m = 0; m < MI; ++m)
 #pragma unroll
-                for (int n = 0; n < NI; ++n) acc[m][n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[m], b[n], acc[m][n], 0, 0, 0);
+                for (int n = 0; n < NI; ++n) acc[m][n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[j & 1][m], b[j & 1][n], acc[m][n], 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
         }
     }
     int * s_pair = (int *) smem;
@@ -138,29 +155,62 @@ template <int BM, int BN, int WM, int WN, int KIND> __global__ __launch_bounds__
                 }
             continue;
         }
-        const float bias = (ok && p.bias) ? p.bias[col] : 0.0f;
+        (void) ok;
+    }
+    if constexpr (KIND <= EXPERTS) {
+        // (everything the stores need is in registers or LDS: a load among them would wait for the stores in front of it)
+#pragma unroll
+        for (int n = 0; n < NI; ++n) asm volatile("" : "+v"(bias[n]));
 #pragma unroll
         for (int m = 0; m < MI; ++m)
 #pragma unroll
-            for (int e = 0; e < 16; ++e) {
-                int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
-                float v = act_apply(p.act_fn, acc[m][n][e] + bias);
-                if (!ok || tok >= n_tok) continue;
-                if constexpr (KIND == EXPERTS) { v *= s_weight[tok - t0]; tok = s_pair[tok - t0]; }
-                st_type(p.y, (size_t) tok * p.ldy + col, p.y_type, v);
-            }
+            for (int n = 0; n < NI; ++n)
+#pragma unroll
+                for (int e = 0; e < 16; ++e) acc[m][n][e] += bias[n];
+        if (p.act_fn) {
+#pragma unroll
+            for (int m = 0; m < MI; ++m)
+#pragma unroll
+                for (int n = 0; n < NI; ++n)
+#pragma unroll
+                    for (int e = 0; e < 16; ++e) acc[m][n][e] = act_apply(p.act_fn, acc[m][n][e]);
+        }
+        auto put = [&](auto * y, bool whole) __attribute__((always_inline)) {
+#pragma unroll
+            for (int m = 0; m < MI; ++m)
+#pragma unroll
+                for (int e = 0; e < 16; ++e) {
+                    const int in = wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
+                    if (!whole && t0 + in >= n_tok) continue;
+                    float w = 1.0f;
+                    int tok = t0 + in;
+                    if constexpr (KIND == EXPERTS) { w = s_weight[in]; tok = s_pair[in]; }
+                    auto * row = y + (size_t) tok * p.ldy + n0 + wn * WN + lr;
+#pragma unroll
+                    for (int n = 0; n < NI; ++n)
+                        if (whole || n0 + wn * WN + n * 32 + lr < p.n_store) st_g(row + n * 32, from_f<std::remove_reference_t<decltype(*y)>>(KIND == EXPERTS ? acc[m][n][e] * w : acc[m][n][e]));
+                }
+        };
+        const bool whole = t0 + BM <= n_tok && n0 + BN <= p.n_store;
+        if (p.y_type == PM_BF16) { if (whole) put((uint16_t *) p.y, true); else put((uint16_t *) p.y, false); }
+        else { if (whole) put((float *) p.y, true); else put((float *) p.y, false); }
     }
 }
 
-template <int BM, int BN, int WM, int WN, int KIND> int launch(GemmP p, hipStream_t st) {
+template <int BM, int BN, int WM, int WN, int STAGES, int KIND> int launch_stages(GemmP p, hipStream_t st) {
     constexpr int threads = BM / WM * (BN / WN) * 64;
     if (KIND != EXPERTS) p.nt = (p.T + BM - 1) / BM;
     p.nn = (p.n_store + BN - 1) / BN;
-    const size_t lds = (size_t) 2 * (BM + BN) * 128;
-    pm_allow_big_lds((const void *) dense_gemm_kernel<BM, BN, WM, WN, KIND>, lds);
+    const size_t lds = (size_t) STAGES * (BM + BN) * 128;
+    pm_allow_big_lds((const void *) dense_gemm_kernel<BM, BN, WM, WN, STAGES, KIND>, lds);
     const int per = (p.nt * p.nn + 7) / 8;
-    hipLaunchKernelGGL((dense_gemm_kernel<BM, BN, WM, WN, KIND>), dim3(per * 8), dim3(threads), lds, st, p);
+    hipLaunchKernelGGL((dense_gemm_kernel<BM, BN, WM, WN, STAGES, KIND>), dim3(per * 8), dim3(threads), lds, st, p);
     return 0;
+}
+// up to one tile per CU: twice the stages hide the memory's latency; more: two tiles share a CU
+template <int KIND> int launch_128(const GemmP & p, hipStream_t st) {
+    if constexpr (KIND != EXPERTS) if ((long) ((p.T + 127) / 128) * ((p.n_store + 127) / 128) <= 256) return launch_stages<128, 128, 64, 64, 4, KIND>(p, st);
+    return launch_stages<128, 128, 64, 64, 2, KIND>(p, st);
 }
 
 } // namespace
@@ -175,7 +225,7 @@ int pm_launch_dense_gemm(const pm_dense_args & a, hipStream_t st) {
     // rounds of the grid x time of a tile: a 256-tile does four times a 128-tile's work on a whole CU in ~3.4x its time (two 128-tiles share a CU)
     const long big = (long) ((a.T + 255) / 256) * ((a.n_store + 255) / 256), small = (long) ((a.T + 127) / 128) * ((a.n_store + 127) / 128);
     const double cb = (double) ((big + 255) / 256) * 1.7, cs = (double) ((small + 511) / 512);
-    return cb <= cs ? launch<256, 256, 128, 64, DENSE>(p, st) : launch<128, 128, 64, 64, DENSE>(p, st);
+    return cb <= cs ? launch_stages<256, 256, 128, 64, 2, DENSE>(p, st) : launch_128<DENSE>(p, st);
 }
 
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st) {
@@ -192,10 +242,10 @@ int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st) {
     p.nt = (int) (pairs / 128 + (a.r.E < pairs ? a.r.E : pairs));                  // (most tiles there can be: every expert's last one may be short)
     p.W = (const uint16_t *) a.up; p.e_stride = a.up_stride; p.X = (const uint16_t *) a.x; p.lda = a.ldx; p.K = a.width_p; p.N = p.n_store = a.ffp; p.y = a.hid; p.ldy = a.ffp;
     p.y_type = PM_BF16; p.act_fn = a.act_fn; p.gather = 1; p.weight = a.r.w;
-    launch<128, 128, 64, 64, EXPERTS>(p, st);
+    launch_128<EXPERTS>(p, st);
     p.W = (const uint16_t *) a.down; p.e_stride = a.down_stride; p.X = (const uint16_t *) a.hid; p.lda = a.ffp; p.K = a.ffp; p.N = a.width_p; p.n_store = a.width; p.y = a.y; p.ldy = a.ldy;
     p.y_type = a.y_type; p.act_fn = PM355_ACT_NONE; p.gather = 0; p.scatter = 1; p.weight = nullptr;
-    return launch<128, 128, 64, 64, EXPERTS>(p, st);
+    return launch_128<EXPERTS>(p, st);
 }
 
 int pm_launch_latent_expand(const pm_latent_expand & x, hipStream_t st) {
@@ -204,7 +254,7 @@ int pm_launch_latent_expand(const pm_latent_expand & x, hipStream_t st) {
     p.pages = x.pages; p.X = (const uint16_t *) x.cache; p.lda = x.ld; p.K = x.kvp; p.H = x.H;
     GemmP k = p;
     k.W = (const uint16_t *) x.Wk; k.T = x.n_pages * PM_PAGE; k.n_store = x.H * x.dim; k.N = pm_dense_pad(k.n_store); k.y = x.K; k.per = x.dim; k.pad = x.dkp;
-    launch<128, 128, 64, 64, KEYS>(k, st);
+    launch_128<KEYS>(k, st);
     p.W = (const uint16_t *) x.Wv; p.T = pm_dense_pad(x.H * x.vrows); p.N = p.n_store = x.n_pages * PM_PAGE; p.y = x.V; p.per = x.vdim; p.rows_h = x.vrows; p.pad = x.dvp;
-    return launch<128, 128, 64, 64, VALUES>(p, st);
+    return launch_128<VALUES>(p, st);
 }
