@@ -44,8 +44,8 @@ def parse():
     ap.add_argument("--cpu-seconds", type=float, default=12.0)
     ap.add_argument("--no-extras", action="store_true", help="skip extra_configs / plugin_decode / the llama_decode CPU baseline")
     ap.add_argument("--tmp", default=os.environ.get("TMPDIR", "/tmp"), help="where the synthetic GGUF files of the plug-in legs go")
-    ap.add_argument("--design", default="", help="kudirax[:size,size]: prefill / decode throughput and kernel rooflines of the layer-described design at a few sizes, beside a "
-                                                 "llama window of equal size, instead of the headline workload")
+    ap.add_argument("--design", default="", help="kudirax[:size,size] | keranex[:size,size]: prefill / decode throughput and kernel rooflines of the layer-described design at a few "
+                                                 "sizes, beside the closest other model of equal size, instead of the headline workload")
     ap.add_argument("--section", default="", help="(internal) run ONE extra leg in this process and print its JSON: prefill_qwen | long_context[:model]")
     return ap.parse_args()
 

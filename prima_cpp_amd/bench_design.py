@@ -247,8 +247,11 @@ LIKE = {"proj": "qkv", "out": "out", "up": "gate|up", "down": "down", "attention
 
 def main(what, steps, warmup):
     name, _, sizes = what.partition(":")
+    if name.lower() == "keranex":
+        from . import bench_keranex
+        return bench_keranex.main(sizes.split(",") if sizes else [], steps, warmup)
     if name.lower() != "kudirax":
-        raise SystemExit(f"--design {name}: kudirax is the design that is measured here")
+        raise SystemExit(f"--design {name}: kudirax and keranex are measured")
     res = {}
     for size in (sizes.split(",") if sizes else list(SIZES)):
         z = SIZES[size]

@@ -19,6 +19,7 @@ struct GemmP {
     const int32_t * tiles, * order; const float * weight; int64_t e_stride; int top, gather, scatter;
     // KEYS: X rows are those of cache pages; VALUES: the rows of W are (tokens become the columns of the output)
     const int32_t * pages; int H, per, rows_h, pad;              // heads, values per head, rows of W per head, padded head size of the output
+    int splits, split_steps;                                     // DENSE: k ranges of so many 64-k steps; with more than one, y = f32 sums [splits][T][ldy] (reduce_kernel)
 };
 
 template <int N> __device__ __forceinline__ void vm_wait() { asm volatile("s_waitcnt vmcnt(%0)" :: "n"(N) : "memory"); }
@@ -30,9 +31,11 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
     const int wm = wave / (BN / WN), wn = wave % (BN / WN);
     // tile order: XCD x = blockIdx % 8 takes a contiguous run of tiles; runs walk blocks of 8 token tiles column by column
     const int nt = KIND == EXPERTS ? __builtin_amdgcn_readfirstlane(ld_g(p.tiles)) : p.nt;      // (the grid has room for the most tiles there can be)
-    const int total = nt * p.nn, per = (total + 7) / 8;
-    const int slot = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    const int tiles = nt * p.nn, total = KIND == DENSE ? tiles * p.splits : tiles, per = (total + 7) / 8;
+    int slot = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if (slot >= total || (int) (blockIdx.x >> 3) >= per) return;
+    const int split = KIND == DENSE ? slot / tiles : 0;
+    slot -= split * tiles;
     const int band = slot / (8 * p.nn), left = nt - band * 8, bh = left < 8 ? left : 8, in = slot - band * 8 * p.nn;
     int t0 = (band * 8 + in % bh) * BM, n_tok = p.T;
     const int n0 = (in / bh) * BN;
@@ -67,9 +70,10 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
             off[i] = (uint32_t) (lane >> 3) * (uint32_t) p.lda * 2u + swz;
         } else off[i] = (uint32_t) row * pitch + swz;
     }
+    const int k0 = KIND == DENSE ? split * p.split_steps : 0;
     auto request = [&](int k, int stage) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < PIECES; ++i) pm_dma16((KIND >= KEYS && paged ? pbase[i] : base) + (size_t) k * 128, off[i], lds0 + (uint32_t) stage * STAGE + (uint32_t) i * 1024u);
+        for (int i = 0; i < PIECES; ++i) pm_dma16((KIND >= KEYS && paged ? pbase[i] : base) + (size_t) (k0 + k) * 128, off[i], lds0 + (uint32_t) stage * STAGE + (uint32_t) i * 1024u);
     };
     f32x16 acc[MI][NI];
 #pragma unroll
@@ -87,7 +91,7 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
     float bias[NI];
 #pragma unroll
     for (int n = 0; n < NI; ++n) { const int col = n0 + wn * WN + n * 32 + lr; bias[n] = KIND == DENSE && p.bias && col < p.n_store ? ld_g(p.bias + col) : 0.0f; }
-    const int steps = p.K >> 6;
+    const int steps = KIND == DENSE && p.split_steps < (p.K >> 6) - k0 ? p.split_steps : (p.K >> 6) - k0;
 #pragma unroll
     for (int i = 0; i < STAGES - 1; ++i) if (i < steps) request(i, i);
     for (int k = 0; k < steps; ++k) {
@@ -134,25 +138,31 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
     for (int n = 0; n < NI; ++n) {
         const int col = n0 + wn * WN + n * 32 + lr;
         const bool ok = col < p.n_store;
+        // (32 rows of the tile lie in one page, or belong to one head)
         if constexpr (KIND == KEYS) {                      // K[page][head][slot][pad]
             const int h = col / p.per, d = col - h * p.per;
 #pragma unroll
-            for (int m = 0; m < MI; ++m)
+            for (int m = 0; m < MI; ++m) {
+                const int tok0 = t0 + wm * WM + m * 32;
+                uint16_t * o = (uint16_t *) p.y + (((size_t) (tok0 / PM_PAGE) * p.H + h) * PM_PAGE + tok0 % PM_PAGE) * p.pad + d;
+                if (!ok || tok0 >= p.T) continue;          // (whole pages)
 #pragma unroll
-                for (int e = 0; e < 16; ++e) {
-                    const int tok = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_;
-                    if (ok && tok < p.T) ((uint16_t *) p.y)[(((size_t) (tok / PM_PAGE) * p.H + h) * PM_PAGE + tok % PM_PAGE) * p.pad + d] = f2bf(acc[m][n][e]);
-                }
+                for (int e = 0; e < 16; ++e) st_g(o + (size_t) ((e & 3) + 8 * (e >> 2) + 4 * h_) * p.pad, f2bf(acc[m][n][e]));
+            }
             continue;
         }
         if constexpr (KIND == VALUES) {                    // V[page][head][pad][slot]: rows of the tile are W's, columns the keys
 #pragma unroll
-            for (int m = 0; m < MI; ++m)
+            for (int m = 0; m < MI; ++m) {
+                const int row0 = t0 + wm * WM + m * 32, h = row0 / p.rows_h, d0 = row0 - h * p.rows_h;
+                uint16_t * o = (uint16_t *) p.y + (((size_t) (col / PM_PAGE) * p.H + h) * p.pad + d0) * PM_PAGE + col % PM_PAGE;
+                if (!ok || h >= p.H) continue;
 #pragma unroll
                 for (int e = 0; e < 16; ++e) {
-                    const int row = t0 + wm * WM + m * 32 + (e & 3) + 8 * (e >> 2) + 4 * h_, h = row / p.rows_h, d = row - h * p.rows_h;
-                    if (ok && row < p.T && d < p.per && h < p.H) ((uint16_t *) p.y)[(((size_t) (col / PM_PAGE) * p.H + h) * p.pad + d) * PM_PAGE + col % PM_PAGE] = f2bf(acc[m][n][e]);
+                    const int in = (e & 3) + 8 * (e >> 2) + 4 * h_;
+                    if (d0 + in < p.per) st_g(o + (size_t) in * PM_PAGE, f2bf(acc[m][n][e]));
                 }
+            }
             continue;
         }
         (void) ok;
@@ -185,7 +195,7 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
                     float w = 1.0f;
                     int tok = t0 + in;
                     if constexpr (KIND == EXPERTS) { w = s_weight[in]; tok = s_pair[in]; }
-                    auto * row = y + (size_t) tok * p.ldy + n0 + wn * WN + lr;
+                    auto * row = y + (size_t) (KIND == DENSE ? split * p.T + tok : tok) * p.ldy + n0 + wn * WN + lr;
 #pragma unroll
                     for (int n = 0; n < NI; ++n)
                         if (whole || n0 + wn * WN + n * 32 + lr < p.n_store) st_g(row + n * 32, from_f<std::remove_reference_t<decltype(*y)>>(KIND == EXPERTS ? acc[m][n][e] * w : acc[m][n][e]));
@@ -197,19 +207,39 @@ template <int BM, int BN, int WM, int WN, int STAGES, int KIND> __global__ __lau
     }
 }
 
+// sums of k ranges -> act(sum + bias)
+__global__ __launch_bounds__(256) void reduce_kernel(const float * part, int splits, int T, int ldp, const float * bias, int act_fn, void * y, int ldy, int y_type, int n_store) {
+    const int quads = ldp / 4;
+    const long i = (long) blockIdx.x * 256 + threadIdx.x;
+    if (i >= (long) T * quads) return;
+    const int t = (int) (i / quads), c = (int) (i - (long) t * quads) * 4;
+    const float * src = part + (size_t) t * ldp + c;
+    f32x4 v = *(const PM_G f32x4 *) src;
+    for (int s = 1; s < splits; s += 4) {                  // four loads at a time
+        f32x4 r[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) r[j] = *(const PM_G f32x4 *) (src + (size_t) (s + j < splits ? s + j : 0) * T * ldp);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) if (s + j < splits) v += r[j];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) if (c + e < n_store) st_type(y, (size_t) t * ldy + c + e, y_type, act_apply(act_fn, v[e] + (bias ? ld_g(bias + c + e) : 0.0f)));
+}
+
 template <int BM, int BN, int WM, int WN, int STAGES, int KIND> int launch_stages(GemmP p, hipStream_t st) {
     constexpr int threads = BM / WM * (BN / WN) * 64;
+    if (p.splits < 1) { p.splits = 1; p.split_steps = p.K >> 6; }
     if (KIND != EXPERTS) p.nt = (p.T + BM - 1) / BM;
     p.nn = (p.n_store + BN - 1) / BN;
     const size_t lds = (size_t) STAGES * (BM + BN) * 128;
     pm_allow_big_lds((const void *) dense_gemm_kernel<BM, BN, WM, WN, STAGES, KIND>, lds);
-    const int per = (p.nt * p.nn + 7) / 8;
+    const int per = (p.nt * p.nn * p.splits + 7) / 8;
     hipLaunchKernelGGL((dense_gemm_kernel<BM, BN, WM, WN, STAGES, KIND>), dim3(per * 8), dim3(threads), lds, st, p);
     return 0;
 }
 // up to one tile per CU: twice the stages hide the memory's latency; more: two tiles share a CU
 template <int KIND> int launch_128(const GemmP & p, hipStream_t st) {
-    if constexpr (KIND != EXPERTS) if ((long) ((p.T + 127) / 128) * ((p.n_store + 127) / 128) <= 256) return launch_stages<128, 128, 64, 64, 4, KIND>(p, st);
+    if constexpr (KIND != EXPERTS) if ((long) ((p.T + 127) / 128) * ((p.n_store + 127) / 128) * (p.splits > 1 ? p.splits : 1) <= 256) return launch_stages<128, 128, 64, 64, 4, KIND>(p, st);
     return launch_stages<128, 128, 64, 64, 2, KIND>(p, st);
 }
 
@@ -224,14 +254,22 @@ int pm_launch_dense_gemm(const pm_dense_args & a, hipStream_t st) {
     p.n_store = a.n_store; p.act_fn = a.act_fn;
     // rounds of the grid x time of a tile: a 256-tile does four times a 128-tile's work on a whole CU in ~3.4x its time (two 128-tiles share a CU)
     const long big = (long) ((a.T + 255) / 256) * ((a.n_store + 255) / 256), small = (long) ((a.T + 127) / 128) * ((a.n_store + 127) / 128);
+    // too few tiles for the chip: ranges of k to different workgroups, their sums to scratch
+    const int steps = a.K >> 6, ldp = (a.n_store + 3) / 4 * 4;
+    const int most = steps / 4 < (int) (256 / small) ? steps / 4 : (int) (256 / small);
+    if (a.split && small <= 128 && most > 1 && (size_t) most * a.T * ldp <= a.split_floats) {
+        p.split_steps = (steps + most - 1) / most; p.splits = (steps + p.split_steps - 1) / p.split_steps;
+        p.y = a.split; p.ldy = ldp; p.y_type = PM_F32; p.bias = nullptr; p.act_fn = PM355_ACT_NONE;
+        launch_128<DENSE>(p, st);
+        hipLaunchKernelGGL(reduce_kernel, dim3((unsigned) (((long) a.T * (ldp / 4) + 255) / 256)), dim3(256), 0, st, a.split, p.splits, a.T, ldp, a.bias, a.act_fn, a.y, a.ldy, a.y_type, a.n_store);
+        return 0;
+    }
     const double cb = (double) ((big + 255) / 256) * 1.7, cs = (double) ((small + 511) / 512);
     return cb <= cs ? launch_stages<256, 256, 128, 64, 2, DENSE>(p, st) : launch_128<DENSE>(p, st);
 }
 
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st) {
-    // (few rows of W: the prompt kernel's grid would leave most of the chip idle)
-    const bool narrow = a.n_store <= 256 && (long) ((a.T + 127) / 128) * ((a.n_store + 127) / 128) < 64;
-    return a.pro || a.group || a.type != PM_BF16 || a.T <= 64 || narrow ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
+    return a.pro || a.group || a.type != PM_BF16 || a.T <= 64 ? pm_launch_dense_small(a, st) : pm_launch_dense_gemm(a, st);
 }
 
 int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st) {
@@ -239,13 +277,15 @@ int pm_launch_experts_gemm(const pm_expert_args & a, hipStream_t st) {
     if (a.type != PM_BF16 || a.T < 1 || a.width_p % 64 || a.ffp % 64 || (int64_t) a.T * a.ldx * 2 >= 1ll << 32 || pairs * a.ffp * 2 >= 1ll << 32) return PM355_E_SHAPE;
     GemmP p = {};
     p.tiles = a.r.tiles; p.order = a.r.order; p.top = a.r.top;
-    p.nt = (int) (pairs / 128 + (a.r.E < pairs ? a.r.E : pairs));                  // (most tiles there can be: every expert's last one may be short)
+    if (a.r.tile != 128 && a.r.tile != 256) return PM355_E_SHAPE;
+    auto go = [&]() { return a.r.tile == 256 ? launch_stages<256, 256, 128, 64, 2, EXPERTS>(p, st) : launch_128<EXPERTS>(p, st); };
+    p.nt = (int) (pairs / a.r.tile + (a.r.E < pairs ? a.r.E : pairs));                  // (most tiles there can be: every expert's last one may be short)
     p.W = (const uint16_t *) a.up; p.e_stride = a.up_stride; p.X = (const uint16_t *) a.x; p.lda = a.ldx; p.K = a.width_p; p.N = p.n_store = a.ffp; p.y = a.hid; p.ldy = a.ffp;
     p.y_type = PM_BF16; p.act_fn = a.act_fn; p.gather = 1; p.weight = a.r.w;
-    launch_128<EXPERTS>(p, st);
+    go();
     p.W = (const uint16_t *) a.down; p.e_stride = a.down_stride; p.X = (const uint16_t *) a.hid; p.lda = a.ffp; p.K = a.ffp; p.N = a.width_p; p.n_store = a.width; p.y = a.y; p.ldy = a.ldy;
     p.y_type = a.y_type; p.act_fn = PM355_ACT_NONE; p.gather = 0; p.scatter = 1; p.weight = nullptr;
-    return launch_128<EXPERTS>(p, st);
+    return go();
 }
 
 int pm_launch_latent_expand(const pm_latent_expand & x, hipStream_t st) {

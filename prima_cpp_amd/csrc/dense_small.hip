@@ -328,7 +328,7 @@ template <typename T> int launch_type(const pm_dense_args & a, const SmallP & p,
     }
     if constexpr (sizeof(T) == 2)
         if (a.T <= 8 && (size_t) a.T * (a.K * 2 + 16) <= LDS_ACT) return rm == 1 ? launch<T, 1, 1, -1>(p, N, 0, st) : launch<T, 1, 2, -1>(p, N, 0, st);
-    const bool wide = N / 32 >= 512 || (sizeof(T) == 2 && a.T > 64 && (long) (N / 32) * ((a.T + 63) / 64) >= 128);
+    const bool wide = N / 32 >= 512;
     if (a.merge) return PM355_E_SHAPE;                     // (pm_dense_merge_ok)
     if (a.T <= 16) return wide ? launch<T, 1, 2, 0>(p, N, 0, st) : launch<T, 1, 1, 0>(p, N, 0, st);
     if (a.T <= 32) return wide ? launch<T, 2, 2, 0>(p, N, 0, st) : launch<T, 2, 1, 0>(p, N, 0, st);
@@ -361,7 +361,8 @@ template <typename T> int experts_type(const pm_expert_args & a, hipStream_t st)
 
 } // namespace
 
-bool pm_dense_merge_ok(int T, int K) { return T <= 8 && (size_t) T * (K * 2 + 16) <= LDS_ACT; }
+// (every workgroup of a head merges that head's sums again: with more tokens a launch of its own costs less)
+bool pm_dense_merge_ok(int T, int K) { return T <= 2 && (size_t) T * (K * 2 + 16) <= LDS_ACT; }
 bool pm_dense_pro_ok(int T, int width) { return T >= 1 && T <= 4 && width * (T == 1 ? 1 : T == 2 ? 2 : 4) <= PRO_MAX; }
 
 int pm_launch_dense_small(const pm_dense_args & a, hipStream_t st) {

@@ -18,7 +18,7 @@ __device__ __forceinline__ void prefix(const int * count, int E, int * off) {
     }
     if (lane == 0) off[E] = carry;
 }
-// which experts have pairs, and their 128-pair tiles; one wave
+// which experts have pairs, and their tiles; one wave
 __device__ __forceinline__ void lists(const int * off, const pm_route & r, int want_tiles) {
     const int lane = threadIdx.x & 63;
     int n_act = 0, n_tile = 0;
@@ -28,12 +28,12 @@ __device__ __forceinline__ void lists(const int * off, const pm_route & r, int w
         if (n > 0) r.active[1 + n_act + __popcll(on & ((1ull << lane) - 1))] = e;
         n_act += __popcll(on);
         if (!want_tiles) continue;
-        const int tiles = (n + 127) / 128;
+        const int tiles = (n + r.tile - 1) / r.tile;
         int s = tiles;
         for (int o = 1; o < 64; o *= 2) { const int u = __shfl_up(s, o); if (lane >= o) s += u; }
         for (int i = 0; i < tiles; ++i) {
             int32_t * t = r.tiles + 1 + 3 * (n_tile + s - tiles + i);
-            t[0] = e; t[1] = off[e] + i * 128; t[2] = n - i * 128 < 128 ? n - i * 128 : 128;
+            t[0] = e; t[1] = off[e] + i * r.tile; t[2] = n - i * r.tile < r.tile ? n - i * r.tile : r.tile;
         }
         n_tile += __shfl(s, 63);
     }

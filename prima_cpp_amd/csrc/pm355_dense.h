@@ -22,6 +22,7 @@ struct pm_add_norm {
 };
 // attention outputs of one head per group that are still split by keys: part [T x head tiles][splits][16 heads][K] sums, ml [..][splits][16][maximum (log2 units), sum]
 struct pm_split_merge { const float * part, * ml; int splits, H; };
+constexpr size_t PM_SPLIT_FLOATS = (size_t) 256 * 128 * 128;
 struct pm_dense_args {
     int type; const void * W; int K, N;                 // N: rows of W that exist (multiple of 64)
     const void * act; int lda; int T;
@@ -31,6 +32,7 @@ struct pm_dense_args {
     // group != 0 (a multiple of 32; the small-batch kernel, any T): one matrix per group of `group` rows (attention heads): group g multiplies the K activations from column
     // g * g_act on, its first g_store rows go to the columns from g * g_out on
     int group, g_act, g_out, g_store;
+    float * split; size_t split_floats;                 // != null: scratch for products whose few tiles are split over k (PM_SPLIT_FLOATS always suffices)
     const pm_split_merge * merge;                       // != null (pm_dense_merge_ok, bf16, group = a head): the activations are merged from key splits on the way in
 };
 int pm_launch_dense(const pm_dense_args & a, hipStream_t st);                    // picks the small-batch or the prompt kernel
@@ -138,8 +140,11 @@ struct pm_route {
     int32_t * off;                          // [E + 1] first sorted pair of an expert
     int32_t * order;                        // [T * top] sorted pairs
     int32_t * active;                       // [1 + E] number of experts with pairs, and which
-    int32_t * tiles;                        // [1 + 3 n] number of 128-pair tiles, then {expert, first sorted pair, pairs} each
+    int32_t * tiles;                        // [1 + 3 n] number of tiles, then {expert, first sorted pair, pairs} each
+    int tile;                               // pairs per tile (pm_expert_tile)
 };
+// pairs per tile of the prompt kernel: large ones where an expert has pairs for more than one
+static inline int pm_expert_tile(int64_t pairs, int E) { return pairs >= 384 * (int64_t) E ? 256 : 128; }
 constexpr int PM_ROUTE_PAIR_MAX = 4, PM_ROUTE_ONE_MAX = 64;      // tokens up to which the pairs go one by one / one workgroup routes and sorts
 void pm_launch_route(const pm_route & r, int T, int want_tiles, hipStream_t st);
 struct pm_expert_args {

@@ -10,7 +10,7 @@
 
 namespace {
 
-constexpr int CONV_TOK = 16, TT = 16;
+constexpr int CONV_TOK = 16, TT = 16;                      // tokens a thread of the convolution walks through in prompts; tokens whose scan inputs lie in LDS at a time
 
 // input `back` tokens before token t of the step, x half of the projections; place i in its portion, position pos
 __device__ __forceinline__ float conv_input(const pm_ssm_layer & a, int t, int c, int back, int i, int pos, int seq) {
@@ -18,8 +18,8 @@ __device__ __forceinline__ float conv_input(const pm_ssm_layer & a, int t, int c
     if (i >= back) return ld_any(a.raw, (size_t) (t - back) * a.ldraw + c, a.raw_type);
     return a.cstate[((size_t) seq * (a.conv - 1) + a.conv - 1 + i - back) * a.innerp + c];
 }
-template <typename T, int TAPS> __global__ __launch_bounds__(256) void conv_kernel(pm_ssm_layer a, pm_batch_dev b, int n_tok) {
-    const int c = blockIdx.y * 256 + threadIdx.x, t0 = blockIdx.x * CONV_TOK;
+template <typename T, int TAPS> __global__ __launch_bounds__(256) void conv_kernel(pm_ssm_layer a, pm_batch_dev b, int n_tok, int per) {
+    const int c = blockIdx.y * 256 + threadIdx.x, t0 = blockIdx.x * per;
     if (c >= a.innerp) return;
     const bool real = c < a.inner;
     const int taps = TAPS ? TAPS : a.conv;
@@ -30,7 +30,7 @@ template <typename T, int TAPS> __global__ __launch_bounds__(256) void conv_kern
 #pragma unroll
         for (int j = 0; j < N; ++j) w[j] = a.conv_w[(size_t) c * taps + j];
     }
-    for (int k = 0; k < CONV_TOK && t0 + k < n_tok; ++k) {
+    for (int k = 0; k < per && t0 + k < n_tok; ++k) {
         const int t = t0 + k;
         float v = bias;
         if (real) {
@@ -235,8 +235,9 @@ __global__ __launch_bounds__(256) void scan_carry_kernel(pm_ssm_layer a, const p
 
 int lanes(const pm_ssm_layer & a) { return a.sp >= 256 ? 64 : a.sp / 4; }
 template <typename T> void conv(const pm_ssm_layer & a, const pm_batch_dev & b, int T_, hipStream_t st) {
-    const dim3 grid((T_ + CONV_TOK - 1) / CONV_TOK, (a.innerp + 255) / 256);
-    auto go = [&](auto kern) { hipLaunchKernelGGL(kern, grid, dim3(256), 0, st, a, b, T_); };
+    const int per = T_ <= 64 ? 1 : CONV_TOK;
+    const dim3 grid((T_ + per - 1) / per, (a.innerp + 255) / 256);
+    auto go = [&](auto kern) { hipLaunchKernelGGL(kern, grid, dim3(256), 0, st, a, b, T_, per); };
     if (a.conv == 4) go(conv_kernel<T, 4>);
     else if (a.conv == 3) go(conv_kernel<T, 3>);
     else if (a.conv == 2) go(conv_kernel<T, 2>);
@@ -247,16 +248,18 @@ template <typename T> void step(const pm_ssm_layer & a, const pm_batch_dev & b, 
     auto go = [&](auto kern) { hipLaunchKernelGGL(kern, dim3(T_, (a.inner + cpb - 1) / cpb), dim3(256), 0, st, a, b, lpc); };
     if (a.sp <= 256) go(step_kernel<T, 1>); else if (a.sp == 512) go(step_kernel<T, 2>); else go(step_kernel<T, 4>);
 }
-template <typename T> void scan(const pm_ssm_layer & a, const pm_scan_chunk * chunks, int n, int multi, hipStream_t st) {
+template <typename T, int PHASE> void scan_phase(const pm_ssm_layer & a, const pm_scan_chunk * chunks, int n, hipStream_t st) {
     const int lpc = lanes(a), cpb = 256 / lpc;
     const size_t lds = (size_t) TT * (3 * cpb + 2 * a.sp) * 4;
-    const dim3 grid(n, (a.inner + cpb - 1) / cpb);
-    auto go = [&](auto kern) { pm_allow_big_lds((const void *) kern, lds); hipLaunchKernelGGL(kern, grid, dim3(256), lds, st, a, chunks, lpc); };
+    auto go = [&](auto kern) { pm_allow_big_lds((const void *) kern, lds); hipLaunchKernelGGL(kern, dim3(n, (a.inner + cpb - 1) / cpb), dim3(256), lds, st, a, chunks, lpc); };
+    if (a.sp <= 256) go(scan_kernel<T, 1, PHASE>); else if (a.sp == 512) go(scan_kernel<T, 2, PHASE>); else go(scan_kernel<T, 4, PHASE>);
+}
+template <typename T> void scan(const pm_ssm_layer & a, const pm_scan_chunk * chunks, int n, int multi, hipStream_t st) {
     if (multi) {
-        if (a.sp <= 256) go(scan_kernel<T, 1, 0>); else if (a.sp == 512) go(scan_kernel<T, 2, 0>); else go(scan_kernel<T, 4, 0>);
+        scan_phase<T, 0>(a, chunks, n, st);
         hipLaunchKernelGGL(scan_carry_kernel, dim3(n, (unsigned) (((size_t) a.inner * a.sp / 4 + 255) / 256)), dim3(256), 0, st, a, chunks);
     }
-    if (a.sp <= 256) go(scan_kernel<T, 1, 1>); else if (a.sp == 512) go(scan_kernel<T, 2, 1>); else go(scan_kernel<T, 4, 1>);
+    scan_phase<T, 1>(a, chunks, n, st);
 }
 
 } // namespace

@@ -62,7 +62,7 @@ struct pm_stack : pm355_model {
     pm355_uploader * up = nullptr; void * stage = nullptr; size_t stage_bytes = 0;
 
     int max_tokens = 0; pm355_page_pool * pool = nullptr; std::vector<int> len;
-    float * x[2] = {}, * y = nullptr, * vfirst = nullptr, * part = nullptr, * logits = nullptr; unsigned * ticket = nullptr;
+    float * x[2] = {}, * y = nullptr, * vfirst = nullptr, * part = nullptr, * ksplit = nullptr, * logits = nullptr; unsigned * ticket = nullptr;
     void * xb = nullptr, * raw = nullptr, * q = nullptr, * hb = nullptr, * fin = nullptr;
     std::map<int, void *> att;                 // attention outputs by width: their zero padding stays valid
     int max_raw = 0, max_q = 0, max_ff = 0, max_vf = 0; size_t part_floats = 0;
@@ -475,7 +475,7 @@ int pm_stack::finalize_pool(int max_tokens_, int n_seq, int64_t pool_tokens) {
     Z(x[0], T * Wp * 4); Z(x[1], T * Wp * 4); Z(y, T * Wp * 4); Z(xb, T * Wp * eb); Z(fin, T * Wp * eb);
     Z(raw, T * max_raw * (d.type == PM_BF16 ? 2 : 4) + (size_t) RAW_F32_MAX * max_raw * 4);
     Z(q, T * max_q * eb + slack); Z(hb, T * std::max(max_ff, 64) * eb); Z(vfirst, T * std::max(max_vf, 1) * 4);
-    Z(part, part_floats * 4); Z(ticket, (size_t) GRAPH_MAX_TOKENS * groups * 4 + 64);
+    Z(part, part_floats * 4); if (T > RAW_F32_MAX && d.type == PM_BF16) Z(ksplit, PM_SPLIT_FLOATS * 4); else ksplit = nullptr; Z(ticket, (size_t) GRAPH_MAX_TOKENS * groups * 4 + 64);
     Z(logits, (size_t) HEAD_ROWS * d.n_vocab * 4);
     meta_ints = 16 + 19 * std::max<size_t>(T, 16) + (size_t) pages * 2 + masks.size() * (4 * (T / 16 + 2) + 2 * (size_t) x_pages);
     Z(meta, meta_ints * 4); Z(table, (size_t) n_seq * seq_pages * 4); Z(last, (size_t) n_seq * 4); Z(prev, (size_t) n_seq * 4); Z(last_out, 64);
@@ -647,7 +647,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
     // W . (residual stream, normed by `pre` where the design norms in front of a sublayer); keep: the activations are read again from xb
     auto from_stream = [&](const Mat & m, const float * pre, bool keep, void * out, int ldo, int otype, int n_store, const float * bias, int act) {
         pm_dense_args a{};
-        a.type = ty; a.W = m.d; a.K = m.Kp; a.N = m.Np; a.T = T; a.y = out; a.ldy = ldo; a.y_type = otype; a.n_store = n_store; a.bias = bias; a.act_fn = act;
+        a.type = ty; a.W = m.d; a.K = m.Kp; a.N = m.Np; a.T = T; a.y = out; a.ldy = ldo; a.y_type = otype; a.n_store = n_store; a.bias = bias; a.act_fn = act; a.split = ksplit; a.split_floats = PM_SPLIT_FLOATS;
         if (pend.on && fuse && !pend.parts) {
             const pm_add_norm pro{x[cur], y, Wp, Wp, pend.w, pend.b, d.norm_eps, d.n_embd, x[cur ^ 1], Wp, rms, pre, keep ? xb : nullptr, Wp};
             a.pro = &pro;
@@ -662,6 +662,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
     auto product = [&](const Mat & m, const void * act, int lda, void * out, int ldo, int otype, int n_store, const float * bias, int rows) {
         pm_dense_args a{};
         a.type = ty; a.W = m.d; a.K = m.Kp; a.N = m.Np; a.act = act; a.lda = lda; a.T = rows; a.y = out; a.ldy = ldo; a.y_type = otype; a.n_store = n_store; a.bias = bias;
+        a.split = ksplit; a.split_floats = PM_SPLIT_FLOATS;
         return pm_launch_dense(a, st);
     };
     auto dense = [&](const Mat & m, const void * act, void * out, int ldo, int otype, int n_store, const float * bias, int rows) { return product(m, act, m.Kp, out, ldo, otype, n_store, bias, rows); };
@@ -774,7 +775,7 @@ int pm_stack::launch(const Step & p, hipStream_t st) {
         pm_expert_args a{};
         a.type = ty; a.T = T; a.width_p = Wp; a.ffp = L.ffp; a.width = d.n_embd; a.up = L.e_up.d; a.down = L.e_down.d; a.up_stride = (int64_t) L.ffp * Wp; a.down_stride = (int64_t) Wp * L.ffp;
         a.act_fn = s.act; a.x = xb; a.ldx = Wp; a.hid = hid;
-        a.r = pm_route{rlog, Ep, s.n_expert, s.n_expert_used, s.n_group, s.n_group_keep, rid, rw, rpos, counts + (size_t) L.moe_index * max_E, roff, rorder, ract, rtiles};
+        a.r = pm_route{rlog, Ep, s.n_expert, s.n_expert_used, s.n_group, s.n_group_keep, rid, rw, rpos, counts + (size_t) L.moe_index * max_E, roff, rorder, ract, rtiles, pm_expert_tile((int64_t) T * s.n_expert_used, s.n_expert)};
         const bool pairs = T <= PM_ROUTE_PAIR_MAX;
         parts = pairs ? 0 : s.n_expert_used; y_type = small ? PM_F32 : PM_BF16;
         a.y = pairs ? (void *) y : yrows; a.ldy = Wp; a.y_type = y_type;
