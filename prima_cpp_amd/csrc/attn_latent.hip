@@ -335,7 +335,7 @@ int stages_for(int ld) {
     return n > 8 ? 8 : n;
 }
 int splits_for(int n, int H, int max_keys) {
-    const int HT = (H + 15) / 16, most = (max_keys + 127) / 128, want = (512 + n * HT - 1) / (n * HT), s = want < most ? want : most;
+    const int HT = (H + 15) / 16, most = (max_keys + 63) / 64, want = (256 + n * HT - 1) / (n * HT), s = want < most ? want : most;
     return s < 1 ? 1 : s > 64 ? 64 : s;
 }
 

@@ -32,6 +32,7 @@ CONFIGS = {
                          latent(heads=16, dim=64, rot_dim=64, vdim=64, q_rank=64, kv_rank=300, size=65, scale=0.1), width=64, vocab=64),
     "huge": config(latent(heads=1, dim=260, rot_dim=12, vdim=300, q_rank=70, kv_rank=1100, size=33, scale=0.06), scan(inner=80, state=300, dt_rank=7, conv=4),
                    latent(heads=2, dim=180, rot_dim=70, vdim=20, q_rank=30, kv_rank=520, size=200, scale=0.06, mlp=moe(3, 2, 1, 1, 600)), width=48, vocab=33),
+    "broad": config(scan(inner=1100, state=24, dt_rank=40), latent(heads=4, dim=72, vdim=136, q_rank=560, kv_rank=250, size=120, mlp=moe(7, 3, 1, 1, 300)), width=600, vocab=140),
     "small": small_config(),
 }
 MODELS = {}
@@ -152,6 +153,9 @@ def test_wide_experts(ff, E, top, dtype):
     want = P.run(c, w, toks)
     for n in (1, 4, 5, 33, 64, 150):
         close(alone(m, toks[:n]), want[:n], dtype)
+    if E == 2:                                             # enough pairs per expert for the large tiles
+        toks = tokens(900, c["vocab"], 6)
+        close(alone(m, toks, (450,)), P.run(c, w, toks), dtype)
     m.close()
 
 

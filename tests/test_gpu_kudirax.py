@@ -35,6 +35,7 @@ CONFIGS = {
     "group": config(layer(heads=20, kv=1, dim=16, vdim=8, size=90), layer(heads=20, kv=1, dim=72, vdim=8, size=7, scale=0.3, cap=25.0), width=64, vocab=64),
     "huge_head": config(layer(heads=1, kv=1, dim=260, vdim=12, size=33, scale=0.06), layer(heads=2, kv=1, dim=8, vdim=12, size=1), width=40, vocab=33),
     "late_mix": config(layer(mix=False, vdim=20), layer(vdim=24), layer(heads=3, kv=1, vdim=64, mix=False, ff=None), layer(heads=6, kv=2, dim=48, vdim=24, size=70, scale=0.5, cap=4.0)),
+    "broad": config(layer(heads=4, kv=2, dim=64, vdim=136, size=90, scale=0.1, ff=1200), width=600, vocab=140),
     "small": small_config(),
 }
 MODELS = {}
